@@ -328,7 +328,8 @@ class SinkAttnArgs(ctypes.Structure):
                 ("T", ctypes.c_int64), ("B", ctypes.c_int32), ("n_tiles", ctypes.c_int32), ("q_tile", ctypes.c_int32),
                 ("H", ctypes.c_int32), ("G", ctypes.c_int32), ("dk", ctypes.c_int32), ("dv", ctypes.c_int32),
                 ("window", ctypes.c_int32), ("keep", ctypes.c_int32), ("ring", ctypes.c_int32), ("scale", ctypes.c_float),
-                ("decode_only", ctypes.c_int32), ("act", ctypes.c_int32), ("partial", ctypes.c_void_p), ("partial_splits", ctypes.c_int32)]
+                ("decode_only", ctypes.c_int32), ("act", ctypes.c_int32), ("partial", ctypes.c_void_p), ("partial_splits", ctypes.c_int32),
+                ("chunk", ctypes.c_int32), ("head_scale", ctypes.c_void_p), ("out_row", ctypes.c_int64)]
 
 
 class RecurrentPrepArgs(ctypes.Structure):
@@ -340,6 +341,31 @@ class RecurrentPrepArgs(ctypes.Structure):
                 ("off_q", ctypes.c_int32), ("off_k", ctypes.c_int32), ("off_v", ctypes.c_int32), ("off_beta", ctypes.c_int32),
                 ("taps", ctypes.c_int32), ("unit", ctypes.c_int32), ("sign", ctypes.c_float), ("q_scale", ctypes.c_float),
                 ("act", ctypes.c_int32), ("qkv_silu", ctypes.c_int32)]
+
+
+class SsmPrepareArgs(ctypes.Structure):
+    """Mirror of ``gbxm_ssm_prepare_args``."""
+    _fields_ = [("y", ctypes.c_void_p), ("y_stride", ctypes.c_int64), ("conv", ctypes.c_void_p), ("bias", ctypes.c_void_p), ("tail", ctypes.c_void_p),
+                ("dt_bias", ctypes.c_void_p), ("rate", ctypes.c_void_p), ("seq", ctypes.c_void_p), ("tok", ctypes.c_void_p), ("out", ctypes.c_void_p),
+                ("dt_out", ctypes.c_void_p), ("T", ctypes.c_int64), ("C", ctypes.c_int32), ("H", ctypes.c_int32), ("taps", ctypes.c_int32),
+                ("off_x", ctypes.c_int32), ("off_dt", ctypes.c_int32), ("move_tail", ctypes.c_int32), ("act", ctypes.c_int32)]
+
+
+class HeadScanArgs(ctypes.Structure):
+    """Mirror of ``gbxm_head_scan_args``."""
+    _fields_ = [("rows", ctypes.c_void_p), ("row_stride", ctypes.c_int64), ("decay", ctypes.c_void_p), ("log_decay", ctypes.c_void_p),
+                ("write", ctypes.c_void_p), ("dt_stride", ctypes.c_int64), ("skip", ctypes.c_void_p), ("state", ctypes.c_void_p), ("out", ctypes.c_void_p),
+                ("seq", ctypes.c_void_p), ("T", ctypes.c_int64), ("B", ctypes.c_int32), ("H", ctypes.c_int32), ("G", ctypes.c_int32), ("dk", ctypes.c_int32),
+                ("dv", ctypes.c_int32), ("off_q", ctypes.c_int32), ("off_k", ctypes.c_int32), ("off_v", ctypes.c_int32), ("scale", ctypes.c_float),
+                ("act", ctypes.c_int32)]
+
+
+class LayerUpdateArgs(ctypes.Structure):
+    """Mirror of ``gbxm_layer_update_args``."""
+    _fields_ = [("x", ctypes.c_void_p), ("branch", ctypes.c_void_p), ("branch_row", ctypes.c_int64), ("cand", ctypes.c_void_p), ("mix", ctypes.c_void_p),
+                ("mix_row", ctypes.c_int64), ("extra", ctypes.c_void_p), ("norm_w", ctypes.c_void_p), ("h", ctypes.c_void_p), ("image", ctypes.c_void_p),
+                ("image_row", ctypes.c_int64), ("T", ctypes.c_int64), ("width", ctypes.c_int32), ("top", ctypes.c_int32), ("replace", ctypes.c_int32),
+                ("eps", ctypes.c_float), ("act", ctypes.c_int32)]
 
 
 def mixers_so_path() -> str:
@@ -367,7 +393,7 @@ def mixers() -> ctypes.CDLL:
         i64, i32, p, f32, sz = ctypes.c_int64, ctypes.c_int32, ctypes.c_void_p, ctypes.c_float, ctypes.c_size_t
         L.gbxm_version.restype = ctypes.c_int
         L.gbxm_last_error.restype = ctypes.c_char_p
-        L.gbxm_embed_scaled.argtypes = [p, p, p, p, i64, i32, f32, i32, p]
+        L.gbxm_embed_scaled.argtypes = [p, p, p, p, i64, i64, i32, f32, i32, p]
         L.gbxm_segment_rmsnorm.argtypes = [p, i64, i64, i32, i32, p, p, f32, i32, p]
         L.gbxm_residual_norm_add.argtypes = [p, p, p, p, p, i64, i32, i32, f32, f32, i32, p]
         L.gbxm_stream_rmsnorm.argtypes = [p, p, p, i64, i32, f32, i32, p]
@@ -388,13 +414,13 @@ def mixers() -> ctypes.CDLL:
         L.gbxm_sink_attention.argtypes = [ctypes.POINTER(SinkAttnArgs), p]
         L.gbxm_sink_attention_tiled.argtypes = [i32, i32, i32, i32]
         L.gbxm_hyper_step.argtypes = [p, p, p, p, p, p, p, p, p, p, i64, i32, i32, i32, f32, i32, p]
-        L.gbxm_glu.argtypes = [p, i64, p, i64, i32, i32, f32, f32, i32, p]
+        L.gbxm_glu.argtypes = [p, i64, p, i64, p, i64, i64, i32, i32, f32, f32, i32, p]
         L.gbxm_route_sigmoid_groups.argtypes = [p, p, p, p, i64, i32, i32, i32, i32, i32, f32, p]
         L.gbxm_expert_glu_act.argtypes = [p, p, p, p, p, i64, i32, i32, i32, i32, i32, i32, f32, p, sz, p]
         L.gbxm_recurrent_prepare.argtypes = [ctypes.POINTER(RecurrentPrepArgs), p]
         L.gbxm_conv_tail_update.argtypes = [p, i64, p, p, i32, i32, i32, i32, p]
         L.gbxm_state_scan.argtypes = [p, i64, p, p, p, i32, i64, i32, i32, i32, i32, i32, p]
-        L.gbxm_head_norm_gate.argtypes = [p, p, i64, p, p, i64, i32, i32, f32, i32, i32, p]
+        L.gbxm_head_norm_gate.argtypes = [p, p, i64, p, p, i64, i64, i32, i32, f32, i32, i32, p]
         L.gbxm_embed_hashed_pair.argtypes = [p, p, p, p, p, p, p, i64, i32, i64, i64, i64, i32, p]
         L.gbxm_norm_token_shift.argtypes = [p, p, p, p, p, p, p, i64, i32, f32, i32, p]
         L.gbxm_branch_norm_add_norm.argtypes = [p, p, p, p, p, p, p, i64, i32, i32, f32, i32, p]
@@ -403,6 +429,12 @@ def mixers() -> ctypes.CDLL:
         L.gbxm_causal_conv_rows.argtypes = [p, i64, p, p, p, p, p, p, i64, i32, i32, i32, p]
         L.gbxm_block_gate_logits.argtypes = [p, p, p, p, i64, i32, i32, i32, i32, p]
         L.gbxm_gated_lru_scan.argtypes = [p, p, i64, i64, p, p, i64, p, p, p, i32, i64, i32, i32, f32, i32, p]
+        L.gbxm_ssm_prepare.argtypes = [ctypes.POINTER(SsmPrepareArgs), p]
+        L.gbxm_head_scan.argtypes = [ctypes.POINTER(HeadScanArgs), p]
+        L.gbxm_gate_group_norm.argtypes = [p, p, i64, p, p, i64, i64, i32, i32, f32, i32, p]
+        L.gbxm_layer_update.argtypes = [ctypes.POINTER(LayerUpdateArgs), p]
+        L.gbxm_router_rows.argtypes = [p, p, p, i64, i32, i32, i32, p]
+        L.gbxm_route_groups.argtypes = [p, i64, p, p, i64, i64, i32, i32, i32, i32, i32, p]
         _mlib = L
     return _mlib
 

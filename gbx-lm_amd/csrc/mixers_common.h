@@ -21,6 +21,31 @@ template <typename T> __device__ __forceinline__ T from_f32(float f);
 template <> __device__ __forceinline__ float from_f32<float>(float f) { return f; }
 template <> __device__ __forceinline__ bf16_t from_f32<bf16_t>(float f) { return f32_to_bf16(f); }
 
+// V neighbouring elements of a row to and from fp32: one 8- or 16-byte access for V = 4 (aligned addresses).
+template <typename T, int V> struct Lanes;
+template <typename T> struct Lanes<T, 1> {
+  static __device__ __forceinline__ void load(const T* p, float* v) { v[0] = to_f32(*p); }
+  static __device__ __forceinline__ void store(T* p, const float* v) { *p = from_f32<T>(v[0]); }
+};
+template <> struct Lanes<float, 4> {
+  static __device__ __forceinline__ void load(const float* p, float* v) {
+    const float4 f = *reinterpret_cast<const float4*>(p);
+    v[0] = f.x; v[1] = f.y; v[2] = f.z; v[3] = f.w;
+  }
+  static __device__ __forceinline__ void store(float* p, const float* v) { *reinterpret_cast<float4*>(p) = float4{v[0], v[1], v[2], v[3]}; }
+};
+template <> struct Lanes<bf16_t, 4> {
+  static __device__ __forceinline__ void load(const bf16_t* p, float* v) {
+    const uint2 u = *reinterpret_cast<const uint2*>(p);
+    v[0] = __uint_as_float(u.x << 16); v[1] = __uint_as_float(u.x & 0xFFFF0000u);
+    v[2] = __uint_as_float(u.y << 16); v[3] = __uint_as_float(u.y & 0xFFFF0000u);
+  }
+  static __device__ __forceinline__ void store(bf16_t* p, const float* v) {
+    *reinterpret_cast<uint2*>(p) = uint2{static_cast<unsigned>(f32_to_bf16(v[0])) | (static_cast<unsigned>(f32_to_bf16(v[1])) << 16),
+                                         static_cast<unsigned>(f32_to_bf16(v[2])) | (static_cast<unsigned>(f32_to_bf16(v[3])) << 16)};
+  }
+};
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
@@ -60,6 +85,13 @@ template <bool FAST> __device__ __forceinline__ float glu_act(float g, float u, 
   return g * sigmoid_<FAST>(g) * u;
 }
 template <bool FAST> __device__ __forceinline__ float log1p_(float x) { if constexpr (FAST) return __logf(1.f + x); else return log1pf(x); }
+
+// First position the row at `pos` sees: its chunk's start (chunks of `chunk` tokens counted from position 0), or the window's, or 0.
+// Never falls as pos grows.
+__host__ __device__ __forceinline__ int first_seen(int pos, int window, int chunk) {
+  if (chunk > 0) return pos - pos % chunk;
+  return window > 0 && pos >= window ? pos - window + 1 : 0;
+}
 
 // floats per (split, row, head) of the key-split partial sums of softmax attention: dv sums padded to a multiple of four (rows stay
 // 16-byte aligned), then two more pairs of which the last holds (running maximum, denominator)

@@ -21,13 +21,13 @@ constexpr int NT = 256, NW = NT / 64;
 
 template <typename T>
 __global__ __launch_bounds__(NT) void embed_kernel(const T* __restrict__ table, const int64_t* __restrict__ tokens, float* __restrict__ x,
-                                                   T* __restrict__ h, int width, float scale) {
+                                                   T* __restrict__ h, int64_t h_row, int width, float scale) {
   const int64_t t = blockIdx.x;
   const T* row = table + tokens[t] * width;
   for (int c = threadIdx.x; c < width; c += NT) {
     const float v = to_f32(row[c]) * scale;
     x[t * width + c] = v;
-    if (h) h[t * width + c] = from_f32<T>(v);
+    if (h) h[t * h_row + c] = from_f32<T>(v);
   }
 }
 
@@ -199,12 +199,12 @@ const char* gbxm_last_error(void) { return g_err; }
     if ((act) == GBXM_BF16) { using T = bf16_t; CALL; } else { using T = float; CALL; } \
   } while (0)
 
-int gbxm_embed_scaled(const void* table, const int64_t* tokens, float* x, void* h, int64_t T_, int32_t width, float scale, int32_t act,
+int gbxm_embed_scaled(const void* table, const int64_t* tokens, float* x, void* h, int64_t h_row, int64_t T_, int32_t width, float scale, int32_t act,
                       void* stream) {
-  if (!act_ok(act) || !table || !tokens || !x || width <= 0 || T_ < 0) return fail(GBXM_ERR_INVALID, "embed_scaled: bad argument");
+  if (!act_ok(act) || !table || !tokens || !x || width <= 0 || T_ < 0 || (h && h_row < width)) return fail(GBXM_ERR_INVALID, "embed_scaled: bad argument");
   if (T_ == 0) return GBXM_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  GBXM_DISPATCH(act, (embed_kernel<T><<<dim3(T_), NT, 0, s>>>(static_cast<const T*>(table), tokens, x, static_cast<T*>(h), width, scale)));
+  GBXM_DISPATCH(act, (embed_kernel<T><<<dim3(T_), NT, 0, s>>>(static_cast<const T*>(table), tokens, x, static_cast<T*>(h), h_row, width, scale)));
   return after_launch("embed_scaled");
 }
 

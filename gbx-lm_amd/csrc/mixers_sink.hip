@@ -2,8 +2,9 @@
 // tables, the parallel-layer stream update and the feed-forward activation.
 //
 //   out[t][h] = gate[t][h] * sum_j p_j v_j,   p_j = exp(s_j) / (exp(sink_h) + sum_j exp(s_j)),   s_j = scale <q[t][h], k_j>
-// over the keys j <= i of the row's sequence with i - j < window or j < keep.  The keys a row sees are two runs of positions,
-// [0, min(keep, lo)) and [lo, i] with lo = max(0, i - window + 1); the kernels walk them as ONE run of indices (no masked key is
+// over the keys j <= i of the row's sequence with i - j < window (or, with chunks instead of a window, j in the same chunk of
+// positions as i) or j < keep; s_j may carry a factor per query head.  The keys a row sees are two runs of positions,
+// [0, min(keep, lo)) and [lo, i] with lo = first_seen(i); the kernels walk them as ONE run of indices (no masked key is
 // ever loaded).  Position j of a sequence is read from its slot's table (row j if j < keep, else keep + (j - keep) % ring) when it
 // lies before the step, and from the step's own rows otherwise.
 //
@@ -26,8 +27,10 @@ constexpr int DCH = 128;          // value channels per lane pass (two per lane)
 constexpr int NCH = 4;            // lane passes: value sizes up to NCH * DCH
 
 struct SinkGeo {
-  int H, G, dk, dv, window, keep, ring;
+  int H, G, dk, dv, window, keep, ring, chunk;
   float scale;
+  const float* head_scale;
+  int64_t out_row;
   int64_t q_row, q_head, k_row, k_head, v_row, v_head, kc_slot, kc_row, kc_head, vc_slot, vc_row, vc_head, gate_row;
 };
 
@@ -91,7 +94,7 @@ __global__ __launch_bounds__(NT) void sink_rows_kernel(const T* __restrict__ q, 
     for (int r = 0; r < RC; ++r) acc[c][r][0] = acc[c][r][1] = 0.f;
   const bool pair_loads = g.dv % 2 == 0 && VEC;
   // the visible keys as one run of indices: [0, na) are positions 0 .. na-1 (kept first tokens that left the window), the rest lo ..
-  const int lo = g.window > 0 ? max(0, pos - g.window + 1) : 0;
+  const int lo = first_seen(pos, g.window, g.chunk);
   const int na = min(g.keep, lo);
   const int total = na + (pos - lo + 1);
   for (int it = static_cast<int>(blockIdx.z) * KT; it < total; it += KT * splits) {
@@ -112,7 +115,7 @@ __global__ __launch_bounds__(NT) void sink_rows_kernel(const T* __restrict__ q, 
     __syncthreads();
     for (int i = threadIdx.x; i < nr * KT; i += NT) {
       const int r = i / KT, jj = i % KT;
-      gl[i] = it + jj < total ? dot_row<T, VEC>(ql + r * g.dk, kptr[jj], g.dk) * g.scale : -INFINITY;
+      gl[i] = it + jj < total ? dot_row<T, VEC>(ql + r * g.dk, kptr[jj], g.dk) * (g.head_scale ? g.scale * g.head_scale[head0 + r] : g.scale) : -INFINITY;
     }
     __syncthreads();
     for (int r = wave; r < nr; r += NW) {           // a wave per head: the tile's maximum, the weights, their sum
@@ -197,7 +200,7 @@ __global__ __launch_bounds__(NT) void sink_rows_kernel(const T* __restrict__ q, 
     }
     return;
   }
-  T* orow = out + t * (static_cast<int64_t>(g.H) * g.dv) + head0 * g.dv;
+  T* orow = out + t * g.out_row + head0 * g.dv;
   for (int i = threadIdx.x; i < nr * g.dv; i += NT) {
     const int r = i / g.dv;
     float s = 0.f;
@@ -214,7 +217,8 @@ __global__ __launch_bounds__(NT) void sink_rows_kernel(const T* __restrict__ q, 
 // reads four channels at once; the two halves of the workgroup take the even and the odd splits and meet in LDS.
 template <typename T, bool FAST>
 __global__ __launch_bounds__(256) void sink_reduce_kernel(const float* __restrict__ partial, T* __restrict__ out, const float* __restrict__ sink,
-                                                         const T* __restrict__ gate, int64_t gate_row, int64_t T_, int H, int dv, int splits) {
+                                                         const T* __restrict__ gate, int64_t gate_row, int64_t T_, int H, int dv, int splits,
+                                                         int64_t out_row) {
   __shared__ float wz[64];
   __shared__ float den;
   __shared__ float4 other[128];
@@ -254,7 +258,7 @@ __global__ __launch_bounds__(256) void sink_reduce_kernel(const float* __restric
     if (!half && d < dv) {
       const float4 u = other[q];
       const float r[4] = {(s.x + u.x) * f, (s.y + u.y) * f, (s.z + u.z) * f, (s.w + u.w) * f};
-      for (int c = 0; c < 4 && d + c < dv; ++c) out[(t * H + head) * dv + d + c] = from_f32<T>(r[c]);
+      for (int c = 0; c < 4 && d + c < dv; ++c) out[t * out_row + head * dv + d + c] = from_f32<T>(r[c]);
     }
   }
 }
@@ -287,7 +291,7 @@ int launch_rows(const gbxm_sink_attn_args& a, const SinkGeo& g, int rc, int chun
     sink_rows_kernel<T, FAST, true><<<grid, NT, lds, s>>>(q, kn, vn, kc, vc, a.seq, a.tok, out, a.sink, gate, g, rc, splits, part);
   else
     sink_rows_kernel<T, FAST, false><<<grid, NT, lds, s>>>(q, kn, vn, kc, vc, a.seq, a.tok, out, a.sink, gate, g, rc, splits, part);
-  if (splits > 1) sink_reduce_kernel<T, FAST><<<dim3(a.T, a.H), 256, 0, s>>>(part, out, a.sink, gate, a.gate_row, a.T, a.H, a.dv, splits);
+  if (splits > 1) sink_reduce_kernel<T, FAST><<<dim3(a.T, a.H), 256, 0, s>>>(part, out, a.sink, gate, a.gate_row, a.T, a.H, a.dv, splits, g.out_row);
   return after_launch("sink_attention (rows)");
 }
 
@@ -522,7 +526,8 @@ bool sink_tiles_shape(int dk, int dv);
 
 int launch_sink_reduce(const gbxm_sink_attn_args& a, int splits, hipStream_t s) {
   sink_reduce_kernel<bf16_t, true><<<dim3(a.T, a.H), 256, 0, s>>>(static_cast<const float*>(a.partial), static_cast<bf16_t*>(a.out), a.sink,
-                                                                  static_cast<const bf16_t*>(a.gate), a.gate_row, a.T, a.H, a.dv, splits);
+                                                                  static_cast<const bf16_t*>(a.gate), a.gate_row, a.T, a.H, a.dv, splits,
+                                                                  a.out_row > 0 ? a.out_row : static_cast<int64_t>(a.H) * a.dv);
   return after_launch("sink_attention (join of key splits)");
 }
 
@@ -635,6 +640,9 @@ int gbxm_sink_attention(const gbxm_sink_attn_args* a, void* stream) {
       (a->kcache && !a->vcache))
     return fail(GBXM_ERR_INVALID, "sink_attention: bad geometry");
   if (a->window > 0 && a->ring < a->window) return fail(GBXM_ERR_INVALID, "sink_attention: a ring shorter than the window");
+  if (a->chunk > 0 && (a->window > 0 || (a->kcache && a->ring < a->chunk)))
+    return fail(GBXM_ERR_INVALID, "sink_attention: chunks exclude a window and need a ring of a chunk's length");
+  if (a->chunk < 0 || (a->out_row > 0 && a->out_row < static_cast<int64_t>(a->H) * a->dv)) return fail(GBXM_ERR_INVALID, "sink_attention: chunk or output stride");
   if (a->T == 0) return GBXM_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (!a->decode_only && a->act == GBXM_BF16 && a->tiles && a->n_tiles > 0) {
@@ -645,7 +653,8 @@ int gbxm_sink_attention(const gbxm_sink_attn_args* a, void* stream) {
     const int rc = launch_sink_group(*a, s);
     if (rc != GBXM_ERR_UNSUPPORTED) return rc;
   }
-  SinkGeo g{a->H, a->G, a->dk, a->dv, a->window, a->keep, a->ring, a->scale, a->q_row, a->q_head, a->k_row, a->k_head, a->v_row, a->v_head,
+  SinkGeo g{a->H, a->G, a->dk, a->dv, a->window, a->keep, a->ring, a->chunk, a->scale, a->head_scale,
+            a->out_row > 0 ? a->out_row : static_cast<int64_t>(a->H) * a->dv, a->q_row, a->q_head, a->k_row, a->k_head, a->v_row, a->v_head,
             a->kc_slot, a->kc_row, a->kc_head, a->vc_slot, a->vc_row, a->vc_head, a->gate_row};
   const int R = a->H / a->G;
   if (a->dv > NCH * DCH) return fail(GBXM_ERR_UNSUPPORTED, "sink_attention: value size %d beyond the row kernel (%d)", a->dv, NCH * DCH);

@@ -31,8 +31,10 @@ struct SinkTileArgs {
   const float* sink;
   const bf16_t* gate;
   int64_t q_row, q_head, k_row, k_head, v_row, v_head, kc_slot, kc_row, kc_head, vc_slot, vc_row, vc_head, gate_row;
-  int q_tile, H, G, dk, dv, window, keep, ring;
+  int q_tile, H, G, dk, dv, window, keep, ring, chunk;
   float scale;
+  const float* head_scale;
+  int64_t out_row;
 };
 
 template <int DK, int DV>
@@ -49,7 +51,6 @@ __device__ __forceinline__ void sink_tile(const SinkTileArgs& a, const int tile,
   const int b = a.tiles[2 * tile], tq = a.tiles[2 * tile + 1];
   const int head = blockIdx.y, kvh = head / (a.H / a.G);
   const int slot = a.seq[4 * b], pos0 = a.seq[4 * b + 1], n = a.seq[4 * b + 2], row0 = a.seq[4 * b + 3];
-  const int W = a.window;
   const int qn = min(a.q_tile, n - tq);                     // queries of this tile
   const int qloc = wave * 32 + r;
   const bool qvalid = qloc < qn;
@@ -70,15 +71,16 @@ __device__ __forceinline__ void sink_tile(const SinkTileArgs& a, const int tile,
 
   // the keys any query of the tile sees, as one run of indices: [0, na) are positions 0 .. na-1, the rest lo .. jlast
   const int qfirst = pos0 + tq, jlast = qfirst + qn - 1;
-  const int lo = W > 0 ? max(0, qfirst - W + 1) : 0;
+  const int lo = first_seen(qfirst, a.window, a.chunk);
   const int na = min(a.keep, lo);
   const int total = na + (jlast - lo + 1);
   auto pos_of = [&](int iv) { return iv < na ? iv : lo + (iv - na); };
   const bool wave_live = wave * 32 < qn;
   const int wq0 = qfirst + wave * 32, wq1 = min(wq0 + 31, jlast);      // positions of this wave's queries
+  const int qlo = first_seen(qpos, a.window, a.chunk), wlo0 = first_seen(wq0, a.window, a.chunk), wlo1 = first_seen(wq1, a.window, a.chunk);
 
   constexpr float LOG2E = 1.4426950408889634f;
-  const float scale2 = a.scale * LOG2E;
+  const float scale2 = (a.head_scale ? a.scale * a.head_scale[head] : a.scale) * LOG2E;
   float m = a.sink ? a.sink[head] * LOG2E : -INFINITY;
   float l = (a.sink && hb == 0) ? 1.f : 0.f;                            // the sink counts once per query
   const unsigned char* vbase = vl + (4 * hb + ((lane >> 2) & 3)) * VROW + (16 * ((lane >> 4) & 1) + 4 * (lane & 3)) * 2;
@@ -126,14 +128,14 @@ __device__ __forceinline__ void sink_tile(const SinkTileArgs& a, const int tile,
     if (it + KT < total) fetch(it + KT);                      // the next tile travels while this one is computed
     // wave-uniform: no key of the tile is seen by a query of this wave
     const int jmin = pos_of(it), jmax = pos_of(min(it + KT, total) - 1);
-    if (!wave_live || jmin > wq1 || (W > 0 && jmax < wq0 - W + 1 && jmin >= a.keep)) continue;
+    if (!wave_live || jmin > wq1 || (jmax < wlo0 && jmin >= a.keep)) continue;
 
     f32x16 st = f32x16{0};
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) st = mfma_bf16(*reinterpret_cast<const u32x4*>(kbase + ks * 32), qf[ks], st);
     // scores in units of ln 2 (the exponentials below are base 2).  Inside the mask -- every key of the tile before every query of the
     // wave, inside every window -- nothing is tested per score.
-    const bool inside = it + KT <= total && jmax <= wq0 && (W <= 0 || wq1 - jmin < W || jmax < a.keep);
+    const bool inside = it + KT <= total && jmax <= wq0 && (jmin >= wlo1 || jmax < a.keep);
     float s[16];
     float mx = -INFINITY;
     if (inside) {
@@ -144,7 +146,7 @@ __device__ __forceinline__ void sink_tile(const SinkTileArgs& a, const int tile,
       for (int e = 0; e < 16; ++e) {
         const int iv = it + 8 * (e >> 2) + 4 * hb + (e & 3);
         const int j = pos_of(iv);
-        const bool seen = qvalid && iv < total && j <= qpos && (W <= 0 || qpos - j < W || j < a.keep);
+        const bool seen = qvalid && iv < total && j <= qpos && (j >= qlo || j < a.keep);
         s[e] = seen ? st[e] * scale2 : -INFINITY;
         mx = fmaxf(mx, s[e]);
       }
@@ -185,7 +187,7 @@ __device__ __forceinline__ void sink_tile(const SinkTileArgs& a, const int tile,
     const int64_t row = row0 + tq + qloc;
     float f = 1.f / l;
     if (a.gate) f *= sigmoid_<true>(to_f32(a.gate[row * a.gate_row + head]));
-    bf16_t* op = a.out + row * (static_cast<int64_t>(a.H) * a.dv) + head * a.dv;
+    bf16_t* op = a.out + row * a.out_row + head * a.dv;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
@@ -229,7 +231,6 @@ __global__ __launch_bounds__(256) void sink_group_kernel(const SinkTileArgs a, c
   const int head = kvh * R + min(hloc, R - 1);
   const int b = tok[2 * t], pos = tok[2 * t + 1];
   const int slot = a.seq[4 * b], pos0 = a.seq[4 * b + 1], row0 = a.seq[4 * b + 3];
-  const int W = a.window;
 
   const int ks0 = SPLITK ? wave * KSW : 0;                              // this wave's steps of the score product: ks0 .. ks0 + KSW - 1
   u32x4 qf[KSW];
@@ -245,7 +246,7 @@ __global__ __launch_bounds__(256) void sink_group_kernel(const SinkTileArgs a, c
 #pragma unroll
   for (int i = 0; i < DTW; ++i) o[i] = f32x16{0};
 
-  const int lo = W > 0 ? max(0, pos - W + 1) : 0;
+  const int lo = first_seen(pos, a.window, a.chunk);
   const int na = min(a.keep, lo);
   const int total = na + (pos - lo + 1);
   auto pos_of = [&](int iv) { return iv < na ? iv : lo + (iv - na); };
@@ -259,7 +260,7 @@ __global__ __launch_bounds__(256) void sink_group_kernel(const SinkTileArgs a, c
   };
 
   constexpr float LOG2E = 1.4426950408889634f;
-  const float scale2 = a.scale * LOG2E;
+  const float scale2 = (a.head_scale ? a.scale * a.head_scale[head] : a.scale) * LOG2E;
   const bool own_sink = a.sink && splits == 1;                          // split key tiles: the sink joins in the reduce
   float m = own_sink ? a.sink[head] * LOG2E : -INFINITY;
   float l = (own_sink && hb == 0) ? 1.f : 0.f;
@@ -377,7 +378,7 @@ __global__ __launch_bounds__(256) void sink_group_kernel(const SinkTileArgs a, c
   }
   float f = 1.f / l;
   if (a.gate) f *= sigmoid_<true>(to_f32(a.gate[t * a.gate_row + head]));
-  bf16_t* op = a.out + t * (static_cast<int64_t>(a.H) * a.dv) + head * a.dv;
+  bf16_t* op = a.out + t * a.out_row + head * a.dv;
 #pragma unroll
   for (int i = 0; i < DTW; ++i) {
     const int dt = wave + 4 * i;
@@ -437,7 +438,7 @@ static bool aligned16(const void* p) { return reinterpret_cast<uintptr_t>(p) % 1
 
 static bool tile_operands(const gbxm_sink_attn_args& a) {
   if ((a.q_row | a.q_head | a.k_row | a.k_head | a.v_row | a.v_head) % 8 || !aligned16(a.q) || !aligned16(a.k_new) || !aligned16(a.v_new) ||
-      !aligned16(a.out))
+      !aligned16(a.out) || a.out_row % 8)
     return false;
   if (a.kcache && ((a.kc_slot | a.kc_row | a.kc_head | a.vc_slot | a.vc_row | a.vc_head) % 8 || !aligned16(a.kcache) || !aligned16(a.vcache))) return false;
   return true;
@@ -447,7 +448,8 @@ static SinkTileArgs tile_args(const gbxm_sink_attn_args& a) {
   return SinkTileArgs{static_cast<const bf16_t*>(a.q), static_cast<const bf16_t*>(a.k_new), static_cast<const bf16_t*>(a.v_new),
                       static_cast<const bf16_t*>(a.kcache), static_cast<const bf16_t*>(a.vcache), a.seq, a.tiles, static_cast<bf16_t*>(a.out), a.sink,
                       static_cast<const bf16_t*>(a.gate), a.q_row, a.q_head, a.k_row, a.k_head, a.v_row, a.v_head, a.kc_slot, a.kc_row, a.kc_head,
-                      a.vc_slot, a.vc_row, a.vc_head, a.gate_row, a.q_tile, a.H, a.G, a.dk, a.dv, a.window, a.keep, a.ring, a.scale};
+                      a.vc_slot, a.vc_row, a.vc_head, a.gate_row, a.q_tile, a.H, a.G, a.dk, a.dv, a.window, a.keep, a.ring, a.chunk, a.scale, a.head_scale,
+                      a.out_row > 0 ? a.out_row : static_cast<int64_t>(a.H) * a.dv};
 }
 
 int launch_sink_tiles(const gbxm_sink_attn_args& a, hipStream_t s) {

@@ -222,7 +222,8 @@ __global__ __launch_bounds__(64 * NW) void state_scan_kernel(const float* __rest
 
 template <typename T, bool FAST>
 __global__ __launch_bounds__(NT) void head_norm_gate_kernel(const float* __restrict__ o, const T* __restrict__ gate, int64_t gate_stride,
-                                                           const float* __restrict__ w, T* __restrict__ out, int H, int dv, float eps, int kind) {
+                                                           const float* __restrict__ w, T* __restrict__ out, int64_t out_row, int H, int dv, float eps,
+                                                           int kind) {
   const int64_t t = blockIdx.x;
   const int lane = threadIdx.x & 63;
   const int h = blockIdx.y * NW + (threadIdx.x >> 6);
@@ -232,11 +233,11 @@ __global__ __launch_bounds__(NT) void head_norm_gate_kernel(const float* __restr
   for (int c = lane; c < dv; c += 64) ss += x[c] * x[c];
   const float r = 1.f / sqrtf(wave_sum(ss) / dv + eps);
   const T* g = gate + t * gate_stride + h * dv;
-  T* y = out + (t * H + h) * dv;
+  T* y = out + t * out_row + h * dv;
   for (int c = lane; c < dv; c += 64) {
     const float z = to_f32(g[c]);
     const float s = sigmoid_<FAST>(z);
-    y[c] = from_f32<T>(x[c] * r * w[c] * (kind == 1 ? z * s : s));
+    y[c] = from_f32<T>(x[c] * r * (w ? w[c] : 1.f) * (kind == 1 ? z * s : s));
   }
 }
 
@@ -320,17 +321,17 @@ int gbxm_state_scan(const float* r, int64_t r_stride, float* state, float* out, 
                : launch_scan<false, 1>(R, B, s, r, r_stride, state, out, seq, H, G, dk, dv);
 }
 
-int gbxm_head_norm_gate(const float* o, const void* gate, int64_t gate_stride, const float* w, void* out, int64_t T_, int32_t H, int32_t dv,
+int gbxm_head_norm_gate(const float* o, const void* gate, int64_t gate_stride, const float* w, void* out, int64_t out_row, int64_t T_, int32_t H, int32_t dv,
                         float eps, int32_t kind, int32_t act, void* stream) {
-  if (!act_ok(act) || !o || !gate || !w || !out || T_ < 0 || H < 1 || dv < 1 || gate_stride < H * dv || (kind != 1 && kind != 2))
+  if (!act_ok(act) || !o || !gate || !out || T_ < 0 || H < 1 || dv < 1 || gate_stride < H * dv || out_row < H * dv || (kind != 1 && kind != 2))
     return fail(GBXM_ERR_INVALID, "head_norm_gate: bad argument");
   if (T_ == 0) return GBXM_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
   const dim3 grid(T_, (H + NW - 1) / NW);
   if (act == GBXM_BF16)
-    head_norm_gate_kernel<bf16_t, false><<<grid, NT, 0, s>>>(o, static_cast<const bf16_t*>(gate), gate_stride, w, static_cast<bf16_t*>(out), H, dv, eps, kind);
+    head_norm_gate_kernel<bf16_t, false><<<grid, NT, 0, s>>>(o, static_cast<const bf16_t*>(gate), gate_stride, w, static_cast<bf16_t*>(out), out_row, H, dv, eps, kind);
   else
-    head_norm_gate_kernel<float, false><<<grid, NT, 0, s>>>(o, static_cast<const float*>(gate), gate_stride, w, static_cast<float*>(out), H, dv, eps, kind);
+    head_norm_gate_kernel<float, false><<<grid, NT, 0, s>>>(o, static_cast<const float*>(gate), gate_stride, w, static_cast<float*>(out), out_row, H, dv, eps, kind);
   return after_launch("head_norm_gate");
 }
 

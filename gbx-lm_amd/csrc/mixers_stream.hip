@@ -121,13 +121,21 @@ void launch_hyper_step(int S, dim3 grid, size_t lds, hipStream_t s, float* X, co
 #undef GBXM_HS
 }
 
-template <typename T, bool FAST>
-__global__ __launch_bounds__(NT) void glu_kernel(const T* __restrict__ gu, int64_t stride, T* __restrict__ out, int F, int kind, float limit,
-                                                float alpha) {
+// V channels per thread and pass; with `scale` row t is also multiplied by scale[t * scale_row] before it is rounded.
+template <typename T, bool FAST, int V>
+__global__ __launch_bounds__(NT) void glu_kernel(const T* __restrict__ gu, int64_t stride, const float* __restrict__ scale, int64_t scale_row,
+                                                T* __restrict__ out, int64_t out_row, int F, int kind, float limit, float alpha) {
   const int64_t t = blockIdx.y;
   const T* g = gu + t * stride;
-  for (int f = blockIdx.x * NT + threadIdx.x; f < F; f += gridDim.x * NT)
-    out[t * F + f] = from_f32<T>(glu_act<FAST>(to_f32(g[f]), to_f32(g[F + f]), kind, limit, alpha));
+  const float m = scale ? scale[t * scale_row] : 1.f;
+  for (int f = (blockIdx.x * NT + threadIdx.x) * V; f < F; f += gridDim.x * NT * V) {
+    float a[V], u[V];
+    Lanes<T, V>::load(g + f, a);
+    Lanes<T, V>::load(g + F + f, u);
+#pragma unroll
+    for (int i = 0; i < V; ++i) a[i] = glu_act<FAST>(a[i], u[i], kind, limit, alpha) * m;
+    Lanes<T, V>::store(out + t * out_row + f, a);
+  }
 }
 
 // One wave per row.  LDS: s [E], c [E] (choice scores; -inf once taken or outside the kept groups), group scores [n_groups].
@@ -219,26 +227,36 @@ int gbxm_hyper_step(float* X, const void* y, const float* y_mix, const float* mi
   return after_launch("hyper_step");
 }
 
-int gbxm_glu(const void* gu, int64_t gu_stride, void* out, int64_t T_, int32_t F, int32_t kind, float limit, float alpha, int32_t act, void* stream) {
-  if (!act_ok(act) || !gu || !out || F <= 0 || gu_stride < 2 * F || T_ < 0 || kind < GBXM_GLU_SILU || kind > GBXM_GLU_SIGMOID)
+int gbxm_glu(const void* gu, int64_t gu_stride, const float* scale, int64_t scale_row, void* out, int64_t out_row, int64_t T_, int32_t F, int32_t kind,
+             float limit, float alpha, int32_t act, void* stream) {
+  if (!act_ok(act) || !gu || !out || F <= 0 || gu_stride < 2 * F || out_row < F || T_ < 0 || kind < GBXM_GLU_SILU || kind > GBXM_GLU_SIGMOID)
     return fail(GBXM_ERR_INVALID, "glu: bad argument");
   if (T_ == 0) return GBXM_OK;
   if (T_ > 65535) {                       // rows ride on grid.y: long steps go in slices
     for (int64_t t0 = 0; t0 < T_; t0 += 65535) {
       const int64_t n = T_ - t0 < 65535 ? T_ - t0 : 65535;
       const size_t el = act == GBXM_BF16 ? 2 : 4;
-      const int rc = gbxm_glu(static_cast<const char*>(gu) + t0 * gu_stride * el, gu_stride, static_cast<char*>(out) + t0 * F * el, n, F, kind, limit,
+      const int rc = gbxm_glu(static_cast<const char*>(gu) + t0 * gu_stride * el, gu_stride, scale ? scale + t0 * scale_row : nullptr, scale_row,
+                              static_cast<char*>(out) + t0 * out_row * el, out_row, n, F, kind, limit,
                               alpha, act, stream);
       if (rc) return rc;
     }
     return GBXM_OK;
   }
   hipStream_t s = static_cast<hipStream_t>(stream);
-  const dim3 grid(min((F + NT - 1) / NT, 64), T_);
-  if (act == GBXM_BF16)
-    glu_kernel<bf16_t, true><<<grid, NT, 0, s>>>(static_cast<const bf16_t*>(gu), gu_stride, static_cast<bf16_t*>(out), F, kind, limit, alpha);
-  else
-    glu_kernel<float, false><<<grid, NT, 0, s>>>(static_cast<const float*>(gu), gu_stride, static_cast<float*>(out), F, kind, limit, alpha);
+  const size_t vb = act == GBXM_BF16 ? 8 : 16;
+  const bool vec = F % 4 == 0 && gu_stride % 4 == 0 && out_row % 4 == 0 && (reinterpret_cast<uintptr_t>(gu) | reinterpret_cast<uintptr_t>(out)) % vb == 0;
+  const int V = vec ? 4 : 1;
+  const dim3 grid(min((F + NT * V - 1) / (NT * V), 64), T_);
+#define GBXM_GLU_LAUNCH(T, FAST, V_)                                                                                                                 \
+  glu_kernel<T, FAST, V_><<<grid, NT, 0, s>>>(static_cast<const T*>(gu), gu_stride, scale, scale_row, static_cast<T*>(out), out_row, F, kind, limit, \
+                                              alpha)
+  if (act == GBXM_BF16) {
+    if (vec) GBXM_GLU_LAUNCH(bf16_t, true, 4); else GBXM_GLU_LAUNCH(bf16_t, true, 1);
+  } else {
+    if (vec) GBXM_GLU_LAUNCH(float, false, 4); else GBXM_GLU_LAUNCH(float, false, 1);
+  }
+#undef GBXM_GLU_LAUNCH
   return after_launch("glu");
 }
 

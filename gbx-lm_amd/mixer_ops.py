@@ -34,16 +34,19 @@ def _f32(t: torch.Tensor, name: str) -> torch.Tensor:
     return t
 
 
-def embed_scaled(table: torch.Tensor, tokens: torch.Tensor, scale: float, image: bool = True):
+def embed_scaled(table: torch.Tensor, tokens: torch.Tensor, scale: float, image=True):
     """(x fp32 [T, W], h in the table's dtype): x = table[tokens] * scale; h is x itself for an fp32 table or when no image is asked
-    for (a model whose first layer norms the stream itself)."""
+    for (a model whose first layer norms the stream itself); a tensor [T, W] of the table's dtype as ``image`` (any row stride): h goes there."""
     act = _act(table, "table")
     t, w = tokens.numel(), table.shape[1]
     tokens = tokens.reshape(-1).to(torch.long).contiguous()
     x = torch.empty((t, w), dtype=torch.float32, device=table.device)
-    h = x if (table.dtype == torch.float32 or not image) else torch.empty((t, w), dtype=table.dtype, device=table.device)
+    if isinstance(image, torch.Tensor):
+        h, _ = _out_rows(image, t, w, table, "embed_scaled")
+    else:
+        h = x if (table.dtype == torch.float32 or not image) else torch.empty((t, w), dtype=table.dtype, device=table.device)
     _lib.check_mixers(_lib.mixers().gbxm_embed_scaled(table.data_ptr(), tokens.data_ptr(), x.data_ptr(), None if h is x else h.data_ptr(),
-                                                     t, w, float(scale), act, _stream(table.device)))
+                                                     max(h.stride(0), w), t, w, float(scale), act, _stream(table.device)))
     return x, h
 
 
@@ -240,9 +243,11 @@ def slot_append(cache, k_rows: torch.Tensor, v_rows: Optional[torch.Tensor], bat
 
 
 def sink_attention(q: torch.Tensor, k_new: torch.Tensor, v_new: torch.Tensor, cache, batch, scale: float, window: Optional[int], keep: int,
-                   sink: Optional[torch.Tensor], gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                   sink: Optional[torch.Tensor], gate: Optional[torch.Tensor] = None, chunk: Optional[int] = None,
+                   head_scale: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Context rows [T, H * dv]; q [T, H, dk], k_new [T, G, dk], v_new [T, G, dv] views with unit channel stride, gate [T, H] or None;
-    ``cache`` (models/cache.py:SlotKVCache, or None for a step without history) holds the positions before the step."""
+    ``cache`` (models/cache.py:SlotKVCache, or None for a step without history) holds the positions before the step.  ``chunk``: a row
+    sees its own chunk of positions only; ``head_scale`` fp32 [H]: a factor of every score per query head; ``out``: rows to write into."""
     act = _act(q, "q")
     t, heads, dk = q.shape
     groups, dv = v_new.shape[1], v_new.shape[2]
@@ -261,7 +266,7 @@ def sink_attention(q: torch.Tensor, k_new: torch.Tensor, v_new: torch.Tensor, ca
         kc, vc = cache.keys, cache.values
         if kc.dtype != q.dtype or kc.shape[0] <= max(batch.slot) or kc.shape[2] < groups * dk or vc.shape[2] < groups * dv:
             raise ValueError("sink_attention: the table does not fit the step")
-        if cache.window is None and cache.ring < longest:
+        if cache.window is None and chunk is None and cache.ring < longest:
             raise ValueError("sink_attention: the table is shorter than the step's longest sequence")
         a.kcache, a.kc_slot, a.kc_row, a.kc_head = kc.data_ptr(), kc.stride(0), kc.stride(1), dk
         a.vcache, a.vc_slot, a.vc_row, a.vc_head = vc.data_ptr(), vc.stride(0), vc.stride(1), dv
@@ -270,9 +275,15 @@ def sink_attention(q: torch.Tensor, k_new: torch.Tensor, v_new: torch.Tensor, ca
         if any(batch.pos0):
             raise ValueError("sink_attention: a step with history needs its table")
         a.keep, a.ring = (keep, window) if window is not None else (0, 1)
+    if chunk is not None and (window is not None or (a.kcache and a.ring < chunk)):
+        raise ValueError("sink_attention: chunks exclude a window and need a table of a chunk's rows")
+    if head_scale is not None and head_scale.numel() != heads:
+        raise ValueError("sink_attention: one score factor per head")
     if window is not None and (a.keep != keep or a.ring < window):
         raise ValueError("sink_attention: the table's kept rows / ring do not fit the mask")
-    out = torch.empty((t, heads * dv), dtype=q.dtype, device=q.device)
+    out, a.out_row = _out_rows(out, t, heads * dv, q, "sink_attention")
+    a.chunk = int(chunk or 0)
+    a.head_scale = _f32(head_scale, "head_scale").data_ptr() if head_scale is not None else None
     a.seq, a.tok = batch.seq.data_ptr(), batch.tok.data_ptr()
     a.tiles = batch.tiles.data_ptr() if batch.tiles is not None and batch.tiles.numel() else None
     a.out = out.data_ptr()
@@ -286,7 +297,8 @@ def sink_attention(q: torch.Tensor, k_new: torch.Tensor, v_new: torch.Tensor, ca
     partial = None
     if t * groups < 256 and t <= 64:                            # few rows: room for key-split partial sums
         # keys of the longest row; launches that are being captured are replayed for longer sequences: size for the table then
-        keys = longest if window is None else min(window + keep, longest)
+        span = window if window is not None else chunk
+        keys = longest if span is None else min(span + keep, longest)
         if torch.cuda.is_current_stream_capturing() and cache is not None:
             keys = cache.rows
         splits = min(64, (keys + 63) // 64)
@@ -330,13 +342,27 @@ def hyper_step_(streams: torch.Tensor, y: Optional[torch.Tensor], y_mix: Optiona
     return h if norm is not None else u
 
 
-def glu(gu: torch.Tensor, kind: str, limit: float = 0.0, alpha: float = 1.702) -> torch.Tensor:
+def _out_rows(out: Optional[torch.Tensor], t: int, n: int, like: torch.Tensor, who: str):
+    """(rows to write [t, n], their row stride): ``out`` checked, or new."""
+    if out is None:
+        out = torch.empty((t, n), dtype=like.dtype, device=like.device)
+    elif out.shape != (t, n) or out.dtype != like.dtype or out.stride(1) != 1 or not out.is_cuda:
+        raise ValueError(f"{who}: output rows do not fit")
+    return out, max(out.stride(0), n)
+
+
+def glu(gu: torch.Tensor, kind: str, limit: float = 0.0, alpha: float = 1.702, row_scale: Optional[torch.Tensor] = None,
+        out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``row_scale`` fp32 [T] (any stride): row t of the result times row_scale[t]; ``out``: rows to write into (any row stride)."""
     act = _act(gu, "gu")
     if gu.dim() != 2 or gu.stride(1) != 1 or gu.shape[1] % 2:
         raise ValueError("glu: rows [T, 2F] with unit inner stride")
     t, f = gu.shape[0], gu.shape[1] // 2
-    out = torch.empty((t, f), dtype=gu.dtype, device=gu.device)
-    _lib.check_mixers(_lib.mixers().gbxm_glu(gu.data_ptr(), gu.stride(0), out.data_ptr(), t, f, _GLU[kind], float(limit), float(alpha), act,
+    if row_scale is not None and (row_scale.dtype != torch.float32 or row_scale.shape != (t,)):
+        raise ValueError("glu: one fp32 factor per row")
+    out, out_row = _out_rows(out, t, f, gu, "glu")
+    _lib.check_mixers(_lib.mixers().gbxm_glu(gu.data_ptr(), gu.stride(0), None if row_scale is None else row_scale.data_ptr(),
+                                            0 if row_scale is None else row_scale.stride(0), out.data_ptr(), out_row, t, f, _GLU[kind], float(limit), float(alpha), act,
                                             _stream(gu.device)))
     return out
 
@@ -415,15 +441,16 @@ def decayed_state_scan(r: torch.Tensor, lay, cache, batch, delta: bool) -> torch
     return out
 
 
-def head_norm_gate(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, heads: int, eps: float, kind: int) -> torch.Tensor:
+def head_norm_gate(o: torch.Tensor, gate: torch.Tensor, weight: Optional[torch.Tensor], heads: int, eps: float, kind: int,
+                   out: Optional[torch.Tensor] = None) -> torch.Tensor:
     act = _act(gate, "gate")
     _f32(o, "o")
     t, n = o.shape
-    if gate.shape != (t, n) or gate.stride(1) != 1 or n % heads or weight.numel() != n // heads:
+    if gate.shape != (t, n) or gate.stride(1) != 1 or n % heads or (weight is not None and weight.numel() != n // heads):
         raise ValueError("head_norm_gate: read-outs, gate and weight do not fit")
-    out = torch.empty((t, n), dtype=gate.dtype, device=o.device)
-    _lib.check_mixers(_lib.mixers().gbxm_head_norm_gate(o.data_ptr(), gate.data_ptr(), gate.stride(0), _f32(weight, "weight").data_ptr(), out.data_ptr(),
-                                                       t, heads, n // heads, float(eps), int(kind), act, _stream(o.device)))
+    out, out_row = _out_rows(out, t, n, gate, "head_norm_gate")
+    _lib.check_mixers(_lib.mixers().gbxm_head_norm_gate(o.data_ptr(), gate.data_ptr(), gate.stride(0),
+                                                       None if weight is None else _f32(weight, "weight").data_ptr(), out.data_ptr(), out_row, t, heads, n // heads, float(eps), int(kind), act, _stream(o.device)))
     return out
 
 
@@ -551,3 +578,126 @@ def gated_lru_scan(u: torch.Tensor, logits: torch.Tensor, lam_sp: torch.Tensor, 
                                                        y.data_ptr(), y.stride(0), state.data_ptr(), out.data_ptr(), batch.seq.data_ptr(), len(batch.slot), t, c, bs,
                                                        float(rate), act, _stream(y.device)))
     return out
+
+
+# ------------------------------------------------------------------------------- one decay per head and token (models/recurrent_mixers.py)
+def ssm_prepare(y: torch.Tensor, off_x: int, off_dt: int, conv: torch.Tensor, bias: Optional[torch.Tensor], dt_bias: torch.Tensor, rate: torch.Tensor,
+                cache, batch):
+    """(x | B | C after convolution, bias and silu [T, C] in the rows' dtype, fp32 [T, 2, H]: log decays, step sizes).  ``conv`` [taps, C].
+    Leaves the convolution's last inputs in the cache."""
+    act = _act(y, "y")
+    t, (taps, c), h = y.shape[0], conv.shape, dt_bias.numel()
+    if y.dim() != 2 or y.stride(1) != 1 or t != batch.total or off_x + c > y.shape[1] or off_dt + h > y.shape[1]:
+        raise ValueError("ssm_prepare: projection rows do not fit the step")
+    if conv.dtype != y.dtype or not conv.is_contiguous() or rate.numel() != h or (bias is not None and bias.numel() != c):
+        raise ValueError("ssm_prepare: taps [taps, C] in the rows' dtype, a bias per channel, a rate per head")
+    tail = cache.tail if taps > 1 else None
+    if taps > 1 and (tail is None or tail.dtype != y.dtype or tuple(tail.shape[1:]) != (taps - 1, c) or tail.shape[0] <= max(batch.slot) or not tail.is_contiguous()):
+        raise ValueError("ssm_prepare: the cache's tails do not fit the convolution or the step's slots")
+    out = torch.empty((t, c), dtype=y.dtype, device=y.device)
+    dt = torch.empty((t, 2, h), dtype=torch.float32, device=y.device)
+    a = _lib.SsmPrepareArgs()
+    a.y, a.y_stride, a.conv, a.bias = y.data_ptr(), max(y.stride(0), y.shape[1]), conv.data_ptr(), None if bias is None else _f32(bias, "bias").data_ptr()
+    a.tail = None if tail is None else tail.data_ptr()
+    a.dt_bias, a.rate = _f32(dt_bias, "dt_bias").data_ptr(), _f32(rate, "rate").data_ptr()
+    a.seq, a.tok, a.out, a.dt_out, a.T = batch.seq.data_ptr(), batch.tok.data_ptr(), out.data_ptr(), dt.data_ptr(), t
+    a.C, a.H, a.taps, a.off_x, a.off_dt, a.move_tail, a.act = c, h, taps, off_x, off_dt, int(batch.decode_only), act
+    _lib.check_mixers(_lib.mixers().gbxm_ssm_prepare(ctypes.byref(a), _stream(y.device)))
+    if taps > 1 and not batch.decode_only:
+        conv_tail_update(y[:, off_x:off_x + c], c, cache, batch)
+    return out, dt
+
+
+def head_state_scan(rows: torch.Tensor, heads: int, groups: int, dk: int, dv: int, off_q: int, off_k: int, off_v: int, cache, batch, scale: float = 1.0,
+                    decay: Optional[torch.Tensor] = None, log_decay: Optional[torch.Tensor] = None, write: Optional[torch.Tensor] = None,
+                    skip: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Read-outs fp32 [T, heads * dv]; leaves the new states in ``cache`` (models/cache.py:SlotStateCache)."""
+    act = _act(rows, "rows")
+    t, state = rows.shape[0], cache.state
+    if rows.dim() != 2 or rows.stride(1) != 1 or t != batch.total or max(off_q + groups * dk, off_k + groups * dk, off_v + heads * dv) > rows.shape[1]:
+        raise ValueError("head_state_scan: rows do not fit the step")
+    if (decay is None) == (log_decay is None) or (decay is not None and decay.numel() != heads):
+        raise ValueError("head_state_scan: a constant decay per head, or a logarithm per row and head")
+    per_row = [x for x in (log_decay, write) if x is not None]
+    if any(x.dtype != torch.float32 or x.shape != (t, heads) or x.stride(1) != 1 or x.stride(0) != per_row[0].stride(0) for x in per_row):
+        raise ValueError("head_state_scan: decays and write factors are fp32 [T, heads] of one row stride")
+    if state is None or state.dtype != torch.float32 or tuple(state.shape[1:]) != (heads, dv, dk) or state.shape[0] <= max(batch.slot) or not state.is_contiguous():
+        raise ValueError("head_state_scan: the cache's states do not fit the mixer or the step's slots")
+    out = torch.empty((t, heads * dv), dtype=torch.float32, device=rows.device)
+    a = _lib.HeadScanArgs()
+    a.rows, a.row_stride = rows.data_ptr(), max(rows.stride(0), rows.shape[1])
+    a.decay = None if decay is None else _f32(decay, "decay").data_ptr()
+    a.log_decay, a.write = (None if x is None else x.data_ptr() for x in (log_decay, write))
+    a.dt_stride = max(per_row[0].stride(0), heads) if per_row else 0
+    a.skip = None if skip is None else _f32(skip, "skip").data_ptr()
+    a.state, a.out, a.seq, a.T, a.B = state.data_ptr(), out.data_ptr(), batch.seq.data_ptr(), t, len(batch.slot)
+    a.H, a.G, a.dk, a.dv, a.off_q, a.off_k, a.off_v, a.scale, a.act = heads, groups, dk, dv, off_q, off_k, off_v, float(scale), act
+    _lib.check_mixers(_lib.mixers().gbxm_head_scan(ctypes.byref(a), _stream(rows.device)))
+    return out
+
+
+def gate_group_norm(o: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, groups: int, eps: float, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    act = _act(z, "z")
+    _f32(o, "o")
+    t, n = o.shape
+    if z.shape != (t, n) or z.stride(1) != 1 or n % groups or weight.numel() != n:
+        raise ValueError("gate_group_norm: read-outs, gate and weight do not fit")
+    out, out_row = _out_rows(out, t, n, z, "gate_group_norm")
+    _lib.check_mixers(_lib.mixers().gbxm_gate_group_norm(o.data_ptr(), z.data_ptr(), max(z.stride(0), n), _f32(weight, "weight").data_ptr(), out.data_ptr(),
+                                                        out_row, t, groups, n // groups, float(eps), act, _stream(o.device)))
+    return out
+
+
+# ------------------------------------------------------------------------------- parallel layers with routed experts
+def layer_update_(x: torch.Tensor, branch: torch.Tensor, cand: Optional[torch.Tensor], mix: Optional[torch.Tensor], norm_w: Optional[torch.Tensor],
+                  eps: float, image: Optional[torch.Tensor], replace: bool) -> Optional[torch.Tensor]:
+    """models/residual.py:layer_update_ as one launch; ``mix`` fp32 [T, >= top]: the first ``top`` columns weigh the candidates."""
+    act = _act(branch, "branch")
+    _f32(x, "x")
+    t, width = x.shape
+    if branch.shape != (t, width) or branch.stride(1) != 1:
+        raise ValueError("layer_update_: the branch is [T, W]")
+    a = _lib.LayerUpdateArgs()
+    a.x, a.branch, a.branch_row, a.top = x.data_ptr(), branch.data_ptr(), max(branch.stride(0), width), 0
+    if cand is not None:
+        if cand.dtype != branch.dtype or cand.dim() != 3 or cand.shape[0] != t or cand.shape[2] != width or not cand.is_contiguous():
+            raise ValueError("layer_update_: candidates [T, top, W] in the activation dtype")
+        if mix.dtype != torch.float32 or mix.shape[0] != t or mix.shape[1] < cand.shape[1] or mix.stride(1) != 1:
+            raise ValueError("layer_update_: a weight per candidate")
+        a.cand, a.top, a.mix, a.mix_row = cand.data_ptr(), cand.shape[1], mix.data_ptr(), max(mix.stride(0), mix.shape[1])
+    h = None
+    if norm_w is not None:
+        if norm_w.numel() != width:
+            raise ValueError("layer_update_: one norm weight per channel")
+        h = torch.empty((t, width), dtype=branch.dtype, device=x.device)
+        a.norm_w, a.h = _f32(norm_w, "norm_w").data_ptr(), h.data_ptr()
+    if image is not None:
+        if image.shape != (t, width) or image.dtype != branch.dtype or image.stride(1) != 1:
+            raise ValueError("layer_update_: image rows do not fit")
+        a.image, a.image_row = image.data_ptr(), max(image.stride(0), width)
+    a.T, a.width, a.replace, a.eps, a.act = t, width, int(bool(replace)), float(eps), act
+    _lib.check_mixers(_lib.mixers().gbxm_layer_update(ctypes.byref(a), _stream(x.device)))
+    return h
+
+
+def route_groups(h: torch.Tensor, router: torch.Tensor, experts: int, top: int, groups):
+    """(idx int32 [T, top], weights fp32 [T, top (+ 1)]).  ``router`` fp32 [experts (+ 1), W]: a row past the experts is a gate's, whose sigmoid
+    is the last weight.  Logits in fp32: few rows one HIP launch, prompt-sized steps the vendor library's product."""
+    act = _act(h, "h")
+    t, rows = h.shape[0], router.shape[0]
+    gate = rows - experts
+    if gate not in (0, 1) or router.shape[1] != h.shape[1]:
+        raise ValueError("route_groups: a router row per expert, at most one more")
+    _f32(router, "router")
+    if t <= 32:
+        h = h.contiguous()
+        logits = torch.empty((t, rows), dtype=torch.float32, device=h.device)
+        _lib.check_mixers(_lib.mixers().gbxm_router_rows(h.data_ptr(), router.data_ptr(), logits.data_ptr(), t, h.shape[1], rows, act, _stream(h.device)))
+    else:
+        logits = torch.matmul(h if h.dtype == torch.float32 else h.float(), router.t())
+    idx = torch.empty((t, top), dtype=torch.int32, device=h.device)
+    w = torch.empty((t, top + gate), dtype=torch.float32, device=h.device)
+    count, keep = groups if groups is not None else (0, 0)
+    _lib.check_mixers(_lib.mixers().gbxm_route_groups(logits.data_ptr(), rows, idx.data_ptr(), w.data_ptr(), top + gate, t, experts, top, count, keep, gate,
+                                                     _stream(h.device)))
+    return idx, w

@@ -7,6 +7,7 @@ activation dtype)."""
 from __future__ import annotations
 
 import math
+from typing import Optional
 
 import torch
 import torch.nn.functional as F
@@ -66,21 +67,27 @@ def gate_mul(gate: torch.Tensor, up: torch.Tensor, kind: str) -> torch.Tensor:
     return (_gate_act(gate.float(), kind) * up.float()).to(up.dtype)
 
 
-def glu_(gu: torch.Tensor, kind: str = "silu", limit: float = 0.0, alpha: float = 1.702) -> torch.Tensor:
+def glu_(gu: torch.Tensor, kind: str = "silu", limit: float = 0.0, alpha: float = 1.702, row_scale: Optional[torch.Tensor] = None,
+         out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Rows ``gu`` [T, 2F] = gate | up  ->  [T, F] in the same dtype, fp32 arithmetic.  ``silu``: g sigmoid(g) u.  ``clamped_swish``:
     g' = min(g, limit), u' = clamp(u, -limit, limit), g' sigmoid(alpha g') (u' + 1).  ``gelu_tanh``: gelu(g) u in the tanh form.
-    ``sigmoid``: sigmoid(g) u."""
+    ``sigmoid``: sigmoid(g) u.  ``row_scale`` fp32 [T]: row t of the result times row_scale[t] before it is rounded; ``out``: rows to write
+    into (any row stride)."""
     if kind not in GLU_KINDS:
         raise ValueError(f"unknown gated activation {kind!r}")
     if gu.is_cuda:
         from .. import mixer_ops as M
-        return M.glu(gu, kind, limit, alpha)
+        return M.glu(gu, kind, limit, alpha, row_scale, out)
     f = gu.shape[-1] // 2
     g, u = gu[..., :f].float(), gu[..., f:].float()
     if kind != "clamped_swish":
-        return (_gate_act(g, kind) * u).to(gu.dtype)
-    g, u = g.clamp(max=limit), u.clamp(min=-limit, max=limit)
-    return (g * torch.sigmoid(alpha * g) * (u + 1.0)).to(gu.dtype)
+        y = _gate_act(g, kind) * u
+    else:
+        g, u = g.clamp(max=limit), u.clamp(min=-limit, max=limit)
+        y = g * torch.sigmoid(alpha * g) * (u + 1.0)
+    if row_scale is not None:
+        y = y * row_scale[:, None]
+    return y.to(gu.dtype) if out is None else out.copy_(y.to(gu.dtype))
 
 
 class GatedDenseFeedForward(nn.Module):

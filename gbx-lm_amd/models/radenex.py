@@ -22,7 +22,7 @@ from .base import BaseModelArgs
 from .feed_forward import DenseFeedForward
 from .residual import StreamRMSNorm, stream_add_, stream_add_norm_
 from .sink_attention import LatentAttention, RotatedValueWindowAttention
-from .step_model import RaggedStepModel
+from .step_model import RaggedStepModel, loop_runs
 
 
 @dataclass
@@ -39,13 +39,7 @@ class ModelArgs(BaseModelArgs):
         return self.architecture.lower()
 
     def layer_runs(self) -> List[int]:
-        n = len(self.layers)
-        if not self.loop:
-            return list(range(n))
-        start, stop, times = int(self.loop["start"]), int(self.loop["stop"]), int(self.loop["times"])
-        if not 0 <= start <= stop <= n or times < 0:
-            raise ValueError("Radenex: loop span outside the layers")
-        return list(range(start)) + list(range(start, stop)) * times + list(range(stop, n))
+        return [i for i, _ in loop_runs(len(self.layers), self.loop)]
 
 
 def _mixer(args: ModelArgs, spec: Dict[str, Any]) -> nn.Module:

@@ -15,7 +15,13 @@ scaled to unit length per head, q times a constant, the decay  g = exp(-rate_h *
 exp(A_h)`` -- and ``beta = sigmoid(b)``.  After the scan each head's read-out is RMS-normalised over its value channels, weighted
 and gated (``head_norm_gate``: silu or sigmoid gate).
 
-Mixers: ``GatedLinearAttention`` (plain write, decay from a low-rank projection, silu output gate), ``LightningAttention`` (plain
+States that decay by ONE number per head and token need no such preparation (``head_state_scan`` reads q, k, v from projection rows as
+they are):  S <- d S + w k v^T,  o = scale S^T q + skip v,  d a constant per head or exp of a logarithm per row and head, w a write
+factor per row and head.  For the state space form ``ssm_prepare`` convolves x | B | C and forms log d = -rate softplus(dt + bias) and
+w = softplus(dt + bias); ``gate_group_norm`` gates its read-out first and normalises it in equal parts afterwards.
+
+Mixers: ``Retention`` (a constant decay per head, heads normalised without a weight, silu gate), ``StateSpaceDual`` (Mamba-2),
+``GatedLinearAttention`` (plain write, decay from a low-rank projection, silu output gate), ``LightningAttention`` (plain
 write, silu on q / k / v, a constant decay per head, all heads normalised together, sigmoid gate) and ``ChannelDeltaRule`` (delta
 write with grouped q / k heads, convolution, unit q / k, low-rank decay and low-rank sigmoid gate).
 
@@ -149,18 +155,93 @@ def decayed_state_scan(r: torch.Tensor, lay: RecurrentLayout, cache: SlotStateCa
     return out.view(t, h * dv)
 
 
-def head_norm_gate(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, heads: int, eps: float, kind: int) -> torch.Tensor:
-    """o fp32 [T, heads * dv], gate [T, heads * dv] (activation dtype, unit inner stride), weight fp32 [dv] ->
-    rms_norm_per_head(o) * weight * (silu | sigmoid)(gate) in the gate's dtype."""
+def head_norm_gate(o: torch.Tensor, gate: torch.Tensor, weight: Optional[torch.Tensor], heads: int, eps: float, kind: int,
+                   out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """o fp32 [T, heads * dv], gate [T, heads * dv] (activation dtype, unit inner stride), weight fp32 [dv] or None (no weight) ->
+    rms_norm_per_head(o) * weight * (silu | sigmoid)(gate) in the gate's dtype; ``out``: rows to write into."""
     if o.is_cuda:
         from .. import mixer_ops as M
-        return M.head_norm_gate(o, gate, weight, heads, eps, kind)
+        return M.head_norm_gate(o, gate, weight, heads, eps, kind, out)
     t = o.shape[0]
     x = o.view(t, heads, -1)
-    x = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * weight.float()
+    x = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+    if weight is not None:
+        x = x * weight.float()
     g = gate.float().reshape(t, heads, -1)
     g = F.silu(g) if kind == GATE_SILU else torch.sigmoid(g)
-    return (x * g).reshape(t, -1).to(gate.dtype)
+    y = (x * g).reshape(t, -1).to(gate.dtype)
+    return y if out is None else out.copy_(y)
+
+
+def ssm_prepare(y: torch.Tensor, off_x: int, off_dt: int, conv: torch.Tensor, bias: Optional[torch.Tensor], dt_bias: torch.Tensor, rate: torch.Tensor,
+                cache: SlotStateCache, batch):
+    """Rows of a state space mixer: y [T, N] projection rows, C = conv.shape[1] channels x | B | C at ``off_x``, one step size per head at
+    ``off_dt``; ``conv`` [taps, C] (activation dtype, the last tap meets the current token), ``bias`` fp32 [C] or None, ``dt_bias``, ``rate``
+    fp32 [H].  Returns (silu(conv + bias) [T, C] in the rows' dtype, fp32 [T, 2, H] = (log decay, write factor)) and leaves the
+    convolution's last inputs in the cache."""
+    if y.is_cuda:
+        from .. import mixer_ops as M
+        return M.ssm_prepare(y, off_x, off_dt, conv, bias, dt_bias, rate, cache, batch)
+    taps, c = conv.shape
+    x = y[:, off_x:off_x + c]
+    out = torch.empty((y.shape[0], c), dtype=torch.float32)
+    r0 = 0
+    for slot, pos0, n in zip(batch.slot, batch.pos0, batch.n_new):
+        before = cache.tail[slot].float() if (pos0 and taps > 1) else torch.zeros((taps - 1, c))
+        if 0 < pos0 < taps - 1:                                        # rows of the tail older than the sequence are not its own
+            before = before.clone()
+            before[:taps - 1 - pos0] = 0
+        ext = torch.cat([before, x[r0:r0 + n].float()])
+        acc = torch.zeros((n, c)) if bias is None else bias.float()[None].repeat(n, 1)
+        for j in range(taps):
+            acc += ext[j:j + n] * conv[j].float()
+        out[r0:r0 + n] = F.silu(acc)
+        r0 += n
+    if taps > 1:
+        conv_tail_update(x, c, cache, batch)
+    w = F.softplus(y[:, off_dt:off_dt + dt_bias.numel()].float() + dt_bias.float())
+    return out.to(y.dtype), torch.stack([-rate.float() * w, w], dim=1)
+
+
+def head_state_scan(rows: torch.Tensor, heads: int, groups: int, dk: int, dv: int, off_q: int, off_k: int, off_v: int, cache: SlotStateCache, batch,
+                    scale: float = 1.0, decay: Optional[torch.Tensor] = None, log_decay: Optional[torch.Tensor] = None,
+                    write: Optional[torch.Tensor] = None, skip: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """rows [T, N] hold q and k (``groups`` heads of ``dk`` channels) and v (``heads`` of ``dv``) at the three offsets; ``decay`` fp32 [heads] or
+    ``log_decay`` fp32 [T, heads]; ``write`` fp32 [T, heads] or None; ``skip`` fp32 [heads] or None.  Runs every sequence of the step from
+    the state its slot holds (zeros at position 0), leaves the new state there, returns the read-outs fp32 [T, heads * dv]."""
+    if rows.is_cuda:
+        from .. import mixer_ops as M
+        return M.head_state_scan(rows, heads, groups, dk, dv, off_q, off_k, off_v, cache, batch, scale, decay, log_decay, write, skip)
+    t, rep = rows.shape[0], heads // groups
+    q = rows[:, off_q:off_q + groups * dk].float().view(t, groups, dk).repeat_interleave(rep, 1)
+    k = rows[:, off_k:off_k + groups * dk].float().view(t, groups, dk).repeat_interleave(rep, 1)
+    v = rows[:, off_v:off_v + heads * dv].float().view(t, heads, dv)
+    d = decay.float()[None].expand(t, heads) if decay is not None else torch.exp(log_decay)
+    u = v if write is None else v * write[:, :, None]
+    out = torch.empty((t, heads, dv), dtype=torch.float32)
+    r0 = 0
+    for slot, pos0, n in zip(batch.slot, batch.pos0, batch.n_new):
+        s = cache.state[slot].transpose(1, 2).clone() if pos0 else torch.zeros((heads, dk, dv))
+        for i in range(r0, r0 + n):
+            s = s * d[i][:, None, None] + k[i][:, :, None] * u[i][:, None, :]
+            out[i] = torch.einsum("hkv,hk->hv", s, q[i])
+        cache.state[slot] = s.transpose(1, 2)
+        r0 += n
+    out = out * scale
+    if skip is not None:
+        out = out + skip.float()[None, :, None] * v
+    return out.view(t, heads * dv)
+
+
+def gate_group_norm(o: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, groups: int, eps: float, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """o fp32 [T, n], z [T, n] (activation dtype), weight fp32 [n]: v = o * silu(z), each of the ``groups`` equal parts of v scaled by its own
+    root mean square, times the weight, in z's dtype; ``out``: rows to write into."""
+    if o.is_cuda:
+        from .. import mixer_ops as M
+        return M.gate_group_norm(o, z, weight, groups, eps, out)
+    v = (o * F.silu(z.float())).view(o.shape[0], groups, -1)
+    y = ((v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps)).view(o.shape) * weight.float()).to(z.dtype)
+    return y if out is None else out.copy_(y)
 
 
 def _pad8(n: int) -> int:
@@ -290,3 +371,79 @@ class ChannelDeltaRule(_RecurrentMixer):
         a = F.linear(y[:, self.off_a1:self.off_a1 + self.decay_rank], self.a2.weight)
         gate = F.linear(y[:, self.off_g1:self.off_g1 + self.gate_rank], self.g2.weight)
         return self._mix(y, a, gate, batch, cache)
+
+
+class Retention(nn.Module):
+    """Linear attention with a fixed decay: q = W_q h, k = W_k h / sqrt(dk), v = W_v h per head; S <- decay_h S + k v^T, o = S^T q; each
+    head's read-out scaled to unit root mean square (no weight), times silu(W_g h); then W_o.  q, k and v are read from the projection
+    rows as they are; 1 / sqrt(dk) meets the read-out (the state is linear in k).
+
+    ``own_projections`` False: the caller forms the projection rows (``in_rows``) and applies W_o to what ``mix`` writes."""
+
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, decay, eps: float, own_projections: bool = True):
+        super().__init__()
+        if len(decay) != heads:
+            raise ValueError("Retention: one decay per head")
+        self.heads, self.dim, self.vdim, self.eps = heads, dim, vdim, float(eps)
+        nq, nv = heads * dim, heads * vdim
+        self.off_k, self.off_v, self.off_gate = nq, 2 * nq, 2 * nq + nv
+        self.in_rows, self.ctx_width = _pad8(self.off_gate + nv), nv
+        if own_projections:
+            self.inp = nn.Linear(width, self.in_rows, bias=False)                        # q | k | v | g (| empty rows)
+            self.o = nn.Linear(nv, width, bias=False)
+        self.register_buffer("decay", torch.tensor([float(d) for d in decay], dtype=torch.float64).to(torch.float32))
+        for p in self.parameters():
+            p.requires_grad_(False)
+
+    def make_cache(self, slots) -> SlotStateCache:
+        return SlotStateCache(self.heads, self.dim, self.vdim, 0, 0, slots)
+
+    def mix(self, y: torch.Tensor, batch, cache: SlotStateCache, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        cache.reserve(y.dtype, y.device)
+        o = head_state_scan(y, self.heads, self.heads, self.dim, self.vdim, 0, self.off_k, self.off_v, cache, batch, self.dim ** -0.5, decay=self.decay)
+        return head_norm_gate(o, y[:, self.off_gate:self.off_gate + self.ctx_width], None, self.heads, self.eps, GATE_SILU, out)
+
+    def forward(self, h: torch.Tensor, batch, cache: SlotStateCache) -> torch.Tensor:
+        return F.linear(self.mix(F.linear(h, self.inp.weight), batch, cache), self.o.weight)
+
+
+class StateSpaceDual(nn.Module):
+    """Mamba-2: W_in h = z | x | B | C | dt; x | B | C pass a causal convolution per channel with a bias and silu; dt <- softplus(dt + bias);
+    per head (reading B / C group h // (heads // groups))  S <- exp(-exp(A_log) dt) S + dt B x^T,  y = S^T C + D x;  y * silu(z) is
+    RMS-normalised in ``norm_groups`` equal parts, times a weight; then W_o.  State of a sequence: S (fp32) and the convolution's last
+    ``taps - 1`` inputs.  ``own_projections`` as in ``Retention``."""
+
+    def __init__(self, width: int, heads: int, vdim: int, state: int, groups: int, taps: int, norm_groups: int, eps: float, own_projections: bool = True):
+        super().__init__()
+        if heads % groups or (heads * vdim) % norm_groups or taps < 1:
+            raise ValueError("StateSpaceDual: heads a multiple of groups, equal parts of the norm, at least one tap")
+        self.heads, self.vdim, self.n, self.groups, self.taps = heads, vdim, state, groups, int(taps)
+        self.norm_groups, self.eps = norm_groups, float(eps)
+        self.inner, self.channels = heads * vdim, heads * vdim + 2 * groups * state
+        self.off_dt = self.inner + self.channels
+        self.in_rows, self.ctx_width = _pad8(self.off_dt + heads), self.inner
+        if own_projections:
+            self.inp = nn.Linear(width, self.in_rows, bias=False)                        # z | x | B | C | dt (| empty rows)
+            self.o = nn.Linear(self.inner, width, bias=False)
+        self.register_buffer("conv", torch.zeros((self.taps, self.channels)))            # activation dtype, a row per tap
+        self.register_buffer("conv_bias", torch.zeros(self.channels, dtype=torch.float32))
+        self.register_buffer("dt_bias", torch.zeros(heads, dtype=torch.float32))
+        self.register_buffer("rate", torch.ones(heads, dtype=torch.float32))             # exp(A_log), formed in 32-bit at load time
+        self.register_buffer("skip", torch.zeros(heads, dtype=torch.float32))            # D
+        self.register_buffer("out_norm", torch.ones(self.inner, dtype=torch.float32))
+        for p in self.parameters():
+            p.requires_grad_(False)
+
+    def make_cache(self, slots) -> SlotStateCache:
+        return SlotStateCache(self.heads, self.n, self.vdim, self.channels if self.taps > 1 else 0, self.taps, slots)
+
+    def mix(self, y: torch.Tensor, batch, cache: SlotStateCache, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        cache.reserve(y.dtype, y.device)
+        xbc, dt = ssm_prepare(y, self.inner, self.off_dt, self.conv, self.conv_bias, self.dt_bias, self.rate, cache, batch)
+        gn = self.groups * self.n
+        o = head_state_scan(xbc, self.heads, self.groups, self.n, self.vdim, self.inner + gn, self.inner, 0, cache, batch,
+                            log_decay=dt[:, 0], write=dt[:, 1], skip=self.skip)
+        return gate_group_norm(o, y[:, :self.inner], self.out_norm, self.norm_groups, self.eps, out)
+
+    def forward(self, h: torch.Tensor, batch, cache: SlotStateCache) -> torch.Tensor:
+        return F.linear(self.mix(F.linear(h, self.inp.weight), batch, cache), self.o.weight)

@@ -1,6 +1,7 @@
 """Updates of the fp32 residual stream and the norms that read it.
 
-Branch-norm form:  x <- x + mult * rms_norm(branch) * weight.  Parallel form: ``stream_add_`` / ``stream_add_norm_``.  Several
+Branch-norm form:  x <- x + mult * rms_norm(branch) * weight.  Parallel form: ``stream_add_`` / ``stream_add_norm_``, and
+``layer_update_`` where one of the sublayers is a weighted sum of candidate rows.  Several
 streams (``hyper_step_``): a sublayer reads a weighted sum of ``s`` streams and its output is written to all of them while a small
 matrix mixes the streams among themselves.  ``StreamRMSNorm`` / ``StreamLayerNorm`` turn stream rows into sublayer inputs.
 Sandwich form (a norm in front of AND behind every sublayer): ``branch_norm_add_norm_`` is the update by a normed branch together
@@ -160,3 +161,23 @@ def normed_pair_mean(a: torch.Tensor, b: torch.Tensor, wa: torch.Tensor, wb: tor
     na = fa * torch.rsqrt(fa.pow(2).mean(-1, keepdim=True) + eps) * wa.float()
     nb = fb * torch.rsqrt(fb.pow(2).mean(-1, keepdim=True) + eps) * wb.float()
     return (0.5 * (na + nb)).to(a.dtype)
+
+
+def layer_update_(x: torch.Tensor, branch: torch.Tensor, cand: Optional[torch.Tensor], mix: Optional[torch.Tensor], norm: Optional["StreamRMSNorm"],
+                  image: Optional[torch.Tensor] = None, replace: bool = False) -> Optional[torch.Tensor]:
+    """v = (x, or 0 with ``replace``) + branch [T, W] + sum_k mix[t, k] cand[t, k] (candidates [T, top, W] with fp32 weights, of which the first
+    ``top`` columns are used; None: no candidates), in fp32; the stream ``x`` becomes v in place.  Then ``norm`` of v in the branch's dtype
+    is returned, and / or v's image in that dtype is written to ``image`` [T, W] (any row stride).  GPU tensors: one launch."""
+    if x.is_cuda:
+        from .. import mixer_ops as M
+        return M.layer_update_(x, branch, cand, mix, None if norm is None else norm.weight, 0.0 if norm is None else norm.eps, image, replace)
+    v = branch.float()
+    if cand is not None:
+        v = v + (cand.float() * mix.float()[:, :cand.shape[1], None]).sum(1)
+    if replace:
+        x.copy_(v)
+    else:
+        x.add_(v)
+    if image is not None:
+        image.copy_(x.to(image.dtype))
+    return None if norm is None else norm(x, branch.dtype)

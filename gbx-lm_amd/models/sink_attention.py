@@ -3,14 +3,17 @@
 The core (``sink_attend``): per query head, scores  s_ij = scale * <q_i, k_j>  over the keys the mask shows, weights
 ``p_ij = exp(s_ij) / (exp(sink_h) + sum_j exp(s_ij))``: the sink is a number per head that joins the denominator and has no value
 (``sink = 0`` adds one to the denominator, no sink is the plain softmax).  The mask is causal, optionally a sliding window
-(``i - j < window``) that keeps the first ``keep`` positions of a sequence visible for ever.  Optionally each head's output is
-multiplied by ``sigmoid(gate[t, h])``.  Keys before the step come from a ``SlotKVCache``, the step's own keys from the step.
+(``i - j < window``) that keeps the first ``keep`` positions of a sequence visible for ever, or chunks (``i // chunk == j // chunk``,
+counted from the sequence's first token).  Optionally a factor per query head on the scores, and each head's output multiplied by
+``sigmoid(gate[t, h])``.  Keys before the step come from a ``SlotKVCache``, the step's own keys from the step.
 Scores, weights and the running sums are 32-bit whatever the activation dtype is.
 
 Mixers:
 
 * ``GatedSinkWindowAttention``: grouped-query attention with biases; weighted q / k norm per head before a partial rotation, unit
   values, sliding window, learned sink per head, a sigmoid output gate per channel.
+* ``ChunkedAttention``: grouped-query attention inside chunks of positions; interleaved rotation of the first channels of a head, a
+  temperature per query head, a sigmoid output gate per head.
 * ``RotatedValueWindowAttention``: grouped-query attention; q and k are rotated (rotate-half pairs over the first ``rot_dims``
   channels, any frequency table) and then set to unit root mean square per head; values are rotated by their own position over all
   of their channels and cached so, a head's output is turned back by the query's position (so a value enters rotated by the
@@ -92,17 +95,21 @@ def rotate_norm_heads_(rows: torch.Tensor, positions: torch.Tensor, segments: Li
         seg.copy_(v.to(rows.dtype))
 
 
-def _attend_one(q, k, v, pos_q, pos_k, scale, window, keep, sink, gate):
+def _attend_one(q, k, v, pos_q, pos_k, scale, window, keep, sink, gate, chunk=None, head_scale=None):
     """q [n, H, dk], k [m, G, dk], v [m, G, dv] fp32 of ONE sequence with their positions -> [n, H, dv] fp32."""
     heads, groups = q.shape[1], k.shape[1]
     rep = heads // groups
     kh = k.transpose(0, 1).repeat_interleave(rep, 0)
     vh = v.transpose(0, 1).repeat_interleave(rep, 0)
     s = torch.matmul(q.transpose(0, 1), kh.transpose(1, 2)) * scale                      # [H, n, m]
+    if head_scale is not None:
+        s = s * head_scale.float()[:, None, None]
     i, j = pos_q[:, None], pos_k[None, :]
     seen = j <= i
     if window is not None:
         seen = seen & ((i - j < window) | (j < keep))
+    if chunk is not None:
+        seen = seen & (i // chunk == j // chunk)
     s = s.masked_fill(~seen[None], float("-inf"))
     top = s.max(-1, keepdim=True).values
     if sink is not None:
@@ -118,15 +125,18 @@ def _attend_one(q, k, v, pos_q, pos_k, scale, window, keep, sink, gate):
 
 
 def sink_attend(q: torch.Tensor, k_new: torch.Tensor, v_new: torch.Tensor, cache: Optional[SlotKVCache], batch, scale: float,
-                window: Optional[int], keep: int, sink: Optional[torch.Tensor], gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                window: Optional[int], keep: int, sink: Optional[torch.Tensor], gate: Optional[torch.Tensor] = None, chunk: Optional[int] = None,
+                head_scale: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """q [T, H, dk], k_new [T, G, dk], v_new [T, G, dv] (views with unit inner stride), gate [T, H] or None -> [T, H * dv].
-    ``cache`` (or None when no sequence of the step has history) holds the positions before the step."""
+    ``cache`` (or None when no sequence of the step has history) holds the positions before the step; with ``chunk`` its table is one
+    of ``window = chunk`` rows.  ``head_scale`` fp32 [H]; ``out``: rows to write into (any row stride)."""
     if q.is_cuda:
         from .. import mixer_ops as M
-        return M.sink_attention(q, k_new, v_new, cache, batch, scale, window, keep, sink, gate)
+        return M.sink_attention(q, k_new, v_new, cache, batch, scale, window, keep, sink, gate, chunk, head_scale, out)
     t, heads, _ = q.shape
     groups, dv = v_new.shape[1], v_new.shape[2]
-    out = torch.empty((t, heads * dv), dtype=q.dtype, device=q.device)
+    if out is None:
+        out = torch.empty((t, heads * dv), dtype=q.dtype, device=q.device)
     r0 = 0
     for slot, pos0, n in zip(batch.slot, batch.pos0, batch.n_new):
         k, v = k_new[r0:r0 + n].float(), v_new[r0:r0 + n].float()
@@ -138,7 +148,7 @@ def sink_attend(q: torch.Tensor, k_new: torch.Tensor, v_new: torch.Tensor, cache
             v = torch.cat([cache.values[slot, rows, :groups * dv].float().view(-1, groups, dv), v])
             pos_k = torch.cat([old, pos_k])
         o = _attend_one(q[r0:r0 + n].float(), k, v, torch.arange(pos0, pos0 + n), pos_k, scale, window, keep, sink,
-                        None if gate is None else gate[r0:r0 + n])
+                        None if gate is None else gate[r0:r0 + n], chunk, head_scale)
         out[r0:r0 + n] = o.reshape(n, heads * dv).to(q.dtype)
         r0 += n
     return out
@@ -262,6 +272,56 @@ class GatedSinkWindowAttention(nn.Module):
                           v_rows.view(t, self.kv_heads, self.vdim), cache, batch, self.scale, self.window, 0, self.sink)
         cache_append(cache, k_rows, v_rows, batch)
         return F.linear(gate_mul(y[:, self.off_gate:self.off_gate + self.ng], ctx, "sigmoid"), self.o.weight, self.o.bias)
+
+
+class ChunkedAttention(nn.Module):
+    """Grouped-query attention inside chunks: q | k | v and one gate logit per head from one projection without biases; channels (2i,
+    2i + 1) of the first ``rot_dims`` of every q and k head turn by position * freq[i]; scores times ``scale`` and the query head's
+    ``temp``; position i sees the keys j <= i of its own chunk of ``chunk`` positions (None: all); plain softmax; head h's output times
+    sigmoid(gate_h).  The table keeps one chunk: a chunk's first token starts over the rows of the chunk before.
+
+    ``own_projections`` False: the caller forms the projection rows (``in_rows`` of them) and applies the output projection to what
+    ``mix`` writes (``ctx_width`` channels), say together with those of a sublayer that reads the same input."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, rot_dims: int, rot_base: float, chunk: Optional[int],
+                 scale: float, own_projections: bool = True):
+        super().__init__()
+        if heads % kv_heads or rot_dims % 2 or rot_dims > dim:
+            raise ValueError("heads must be a multiple of kv_heads; the rotated channel count is even and within the head")
+        if chunk is not None and int(chunk) < 1:
+            raise ValueError("ChunkedAttention: chunks hold at least one position")
+        self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
+        self.chunk, self.scale, self.rot_dims = (None if chunk is None else int(chunk)), float(scale), int(rot_dims)
+        self.nq, self.nk, self.nv = heads * dim, kv_heads * dim, kv_heads * vdim
+        self.off_gate = self.nq + self.nk + self.nv
+        self.in_rows, self.ctx_width = (self.off_gate + heads + 7) // 8 * 8, heads * vdim
+        if own_projections:
+            self.inp = nn.Linear(width, self.in_rows, bias=False)                        # q | k | v | g (| empty rows)
+            self.o = nn.Linear(self.ctx_width, width, bias=False)
+        self.register_buffer("freq", rotary_table(rot_base, rot_dims, None)[0] if rot_dims else torch.zeros(0))
+        self.register_buffer("temp", torch.ones(heads))
+        for p in self.parameters():
+            p.requires_grad_(False)
+
+    def make_cache(self, slots) -> SlotKVCache:
+        return SlotKVCache(self.nk, self.nv, self.chunk, 0, slots)
+
+    def mix(self, y: torch.Tensor, batch, cache: SlotKVCache, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        t = y.shape[0]
+        if self.rot_dims:
+            rotate_norm_heads_(y, batch.tok[:, 1], [
+                HeadSegment(0, self.heads, self.dim, 0, self.rot_dims, self.freq, interleaved=True),
+                HeadSegment(self.nq, self.kv_heads, self.dim, 0, self.rot_dims, self.freq, interleaved=True)], 0.0)
+        cache.reserve(max(p + n for p, n in zip(batch.pos0, batch.n_new)), y.dtype, y.device)
+        k_rows, v_rows = y[:, self.nq:self.nq + self.nk], y[:, self.nq + self.nk:self.off_gate]
+        ctx = sink_attend(y[:, :self.nq].unflatten(1, (self.heads, self.dim)), k_rows.unflatten(1, (self.kv_heads, self.dim)),
+                          v_rows.unflatten(1, (self.kv_heads, self.vdim)), cache, batch, self.scale, None, 0, None,
+                          y[:, self.off_gate:self.off_gate + self.heads], self.chunk, self.temp, out)
+        cache_append(cache, k_rows, v_rows, batch)
+        return ctx
+
+    def forward(self, h: torch.Tensor, batch, cache: SlotKVCache) -> torch.Tensor:
+        return F.linear(self.mix(F.linear(h, self.inp.weight), batch, cache), self.o.weight)
 
 
 class LatentAttention(nn.Module):

@@ -8,7 +8,7 @@ it as for any other model.
 """
 from __future__ import annotations
 
-from typing import Any, List
+from typing import Any, Dict, List, Optional, Tuple
 
 import torch
 import torch.nn.functional as F
@@ -16,6 +16,18 @@ from torch import nn
 
 from ..batching import StepBatch
 from .cache import SequenceSlots
+
+
+def loop_runs(n_layers: int, loop: Optional[Dict[str, int]]) -> List[Tuple[int, bool]]:
+    """(layer, whether a pass of the looped span starts with this run) in running order: layers ``start .. stop-1`` run ``times`` times in
+    a row with the same weights, the others once."""
+    if not loop:
+        return [(i, False) for i in range(n_layers)]
+    start, stop, times = int(loop["start"]), int(loop["stop"]), int(loop["times"])
+    if not 0 <= start <= stop <= n_layers or times < 0:
+        raise ValueError("loop span outside the layers")
+    return ([(i, False) for i in range(start)] + [(i, i == start) for _ in range(times) for i in range(start, stop)]
+            + [(i, False) for i in range(stop, n_layers)])
 
 
 class RaggedStepModel(nn.Module):

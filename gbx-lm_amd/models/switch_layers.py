@@ -122,18 +122,23 @@ class DenseRoutedGLU(nn.Module):
 
     Router, ``scoring = "softmax"``: logits in fp32 (``router`` is kept in fp32), probabilities = softmax over ALL experts, the
     ``top`` largest are chosen (ties: the lower expert index); their mixing weights are those probabilities, divided by their sum
-    only if ``renormalize``.  ``scoring = "sigmoid"``: scores s = sigmoid(logits); the choice runs on s + ``correction`` (a vector per
+    only if ``renormalize``; with ``groups = (count, keep)`` (not together with ``renormalize``) the experts form ``count`` equal groups of
+    neighbours, a group's score is its largest probability and only experts of the ``keep`` best groups can be chosen; with ``gate_row`` the
+    router has one more row, the logit of a gate (say of an expert that every token takes): its sigmoid is one more weight, the last
+    column.  ``scoring = "sigmoid"``: scores s = sigmoid(logits); the choice runs on s + ``correction`` (a vector per
     expert that steers the choice and never the weights); with ``groups = (count, keep)`` the experts form ``count`` equal groups of
     neighbours, a group's score is the sum of its two largest choice scores and only experts of the ``keep`` best groups can be
     chosen; weights = the chosen s, divided by their sum (+ 1e-20) if ``renormalize``, times ``route_scale``.
     Expert e: down_e(act(gate_e h, up_e h)); ``activation = "silu"``: silu(g) u; ``"clamped_swish"``: g' = min(g, limit), u' =
     clamp(u, -limit, limit), g' sigmoid(1.702 g') (u' + 1).  ``gate_up`` stacks gate_e over up_e as [E, 2F, K], ``down`` is [E, K, F].
-    ``forward`` returns (y [T, top, K], weights fp32 [T, top]): the weighted sum is left to the caller, which folds it into its
+    ``forward`` returns (y [T, top, K], weights fp32 [T, top], or [T, top + 1] with ``gate_row``): the weighted sum is left to the caller, which folds it into its
     normalisation / residual launch."""
 
     def __init__(self, input_dims: int, hidden_dims: int, num_experts: int, top: int, renormalize: bool = False, scoring: str = "softmax",
-                 groups=None, route_scale: float = 1.0, activation: str = "silu", limit: float = 0.0):
+                 groups=None, route_scale: float = 1.0, activation: str = "silu", limit: float = 0.0, gate_row: bool = False):
         super().__init__()
+        if (gate_row or groups is not None) and scoring == "softmax" and renormalize or (gate_row and scoring != "softmax"):
+            raise ValueError("softmax groups and a gate row go with probabilities as they are")
         if not 1 <= top <= num_experts:
             raise ValueError("top must lie in 1..num_experts")
         if scoring not in ("softmax", "sigmoid") or activation not in ("silu", "clamped_swish"):
@@ -142,8 +147,8 @@ class DenseRoutedGLU(nn.Module):
             raise ValueError("groups: equal groups, 1 <= keep <= count, and the kept groups hold at least top experts")
         self.input_dims, self.hidden_dims, self.num_experts, self.top, self.renormalize = input_dims, hidden_dims, num_experts, top, renormalize
         self.scoring, self.groups, self.route_scale = scoring, (None if groups is None else (int(groups[0]), int(groups[1]))), float(route_scale)
-        self.activation, self.limit = activation, float(limit)
-        self.register_buffer("router", torch.zeros((num_experts, input_dims), dtype=torch.float32))
+        self.activation, self.limit, self.gate_row = activation, float(limit), bool(gate_row)
+        self.register_buffer("router", torch.zeros((num_experts + int(self.gate_row), input_dims), dtype=torch.float32))
         if scoring == "sigmoid":
             self.register_buffer("correction", torch.zeros(num_experts, dtype=torch.float32))
         self.register_buffer("gate_up", torch.zeros((num_experts, 2 * hidden_dims, input_dims)))
@@ -154,6 +159,8 @@ class DenseRoutedGLU(nn.Module):
             from .. import mixer_ops as M
             if self.scoring == "sigmoid":
                 return M.route_sigmoid_groups(h, self.router, self.correction, self.top, self.groups, self.renormalize, self.route_scale)
+            if self.groups is not None or self.gate_row:
+                return M.route_groups(h, self.router, self.num_experts, self.top, self.groups)
             return M.route_topk(h, self.router, self.top, self.renormalize)
         logits = F.linear(h.float(), self.router.float())
         if self.scoring == "sigmoid":
@@ -171,9 +178,19 @@ class DenseRoutedGLU(nn.Module):
             if self.renormalize:
                 w = w / (w.sum(-1, keepdim=True) + 1e-20)
             return idx.to(torch.int32), w * self.route_scale
+        gate, logits = logits[:, self.num_experts:], logits[:, :self.num_experts]
         probs = torch.softmax(logits, dim=-1)
-        w, idx = torch.sort(probs, dim=-1, descending=True, stable=True)      # of equal experts the lower index first
-        w, idx = w[..., :self.top], idx[..., :self.top]
+        c = logits
+        if self.groups is not None:
+            count, keep = self.groups
+            per = c.view(c.shape[0], count, -1)
+            best = torch.sort(per.max(-1).values, dim=-1, descending=True, stable=True).indices[:, :keep]
+            allowed = torch.zeros(per.shape[:2], dtype=torch.bool).scatter_(1, best, True)
+            c = torch.where(allowed[:, :, None].expand_as(per), per, torch.full_like(per, float("-inf"))).reshape(c.shape)
+        idx = torch.sort(c, dim=-1, descending=True, stable=True).indices[..., :self.top]      # of equal experts the lower index first
+        w = torch.gather(probs, 1, idx)
+        if self.gate_row:
+            return idx.to(torch.int32), torch.cat([w, torch.sigmoid(gate)], dim=1)
         if self.renormalize:
             w = w / w.sum(-1, keepdim=True)
         return idx.to(torch.int32), w

@@ -22,8 +22,9 @@ extern "C" {
 int gbxm_version(void);
 const char* gbxm_last_error(void);
 
-/* x[t] = table[token[t]] * scale (fp32 stream) and its image h in the activation dtype (h may be null: no image is written). */
-int gbxm_embed_scaled(const void* table, const int64_t* tokens, float* x, void* h, int64_t T, int32_t width, float scale,
+/* x[t] = table[token[t]] * scale (fp32 stream) and its image h in the activation dtype (rows h_row elements apart; h may be null:
+ * no image is written). */
+int gbxm_embed_scaled(const void* table, const int64_t* tokens, float* x, void* h, int64_t h_row, int64_t T, int32_t width, float scale,
                       int32_t act, void* stream);
 /* In place: rows[t][0:n0] and rows[t][n0:n0+n1] each RMS-normalised over the whole segment (fp32 statistics), times w0 / w1. */
 int gbxm_segment_rmsnorm(void* rows, int64_t T, int64_t row_stride, int32_t n0, int32_t n1, const float* w0, const float* w1,
@@ -110,7 +111,8 @@ int gbxm_slot_append(const void* k, int64_t k_stride, int32_t k_width, const voi
                      void* vcache, const int32_t* seq, const int32_t* tok, int64_t T, int32_t keep, int32_t ring, int32_t act, void* stream);
 
 /* out[t][h] = gate * sum_j p_j v_j,  p_j = exp(s_j) / (exp(sink_h) + sum_j exp(s_j)),  s_j = scale <q[t][h], k_j> over the keys
- * j <= i of the row's sequence with i - j < window or j < keep.  Keys before the step's first row come from the slot tables, the
+ * j <= i of the row's sequence with i - j < window -- or, with chunk > 0 (then window <= 0), floor(i / chunk) = floor(j / chunk) -- or
+ * j < keep; s_j is also multiplied by head_scale[h] if given.  Keys before the step's first row come from the slot tables, the
  * step's own from k_new / v_new.  Strides in elements; the channel stride is 1 everywhere. */
 typedef struct {
   const void* q;      int64_t q_row, q_head;          /* [T][H] x dk */
@@ -133,6 +135,9 @@ typedef struct {
   int32_t decode_only, act;
   void* partial;                /* optional fp32 [partial_splits][T][H][(dv + 3) / 4 * 4 + 4] */
   int32_t partial_splits;
+  int32_t chunk;                /* > 0: a row sees its own chunk of positions only (counted from position 0 of the sequence) */
+  const float* head_scale;      /* [H], or null */
+  int64_t out_row;              /* elements between output rows (0: H*dv) */
 } gbxm_sink_attn_args;
 int gbxm_sink_attention(const gbxm_sink_attn_args* a, void* stream);
 int gbxm_sink_attention_tiled(int32_t dk, int32_t dv, int32_t act, int32_t decode_only);
@@ -148,13 +153,15 @@ int gbxm_sink_attention_tiled(int32_t dk, int32_t dv, int32_t act, int32_t decod
 int gbxm_hyper_step(float* X, const void* y, const float* y_mix, const float* mix, const float* write, const float* read, const float* norm_w,
                     const float* norm_b, void* h, float* out_u, int64_t T, int32_t S, int32_t width, int32_t top, float eps, int32_t act,
                     void* stream);
-/* out[t][f] = act(gu[t][f], gu[t][F + f]) in fp32, rows of 2F in, F out (unit inner strides, row strides in elements).
+/* out[t][f] = act(gu[t][f], gu[t][F + f]) (* scale[t * scale_row] if given) in fp32, rows of 2F in, F out (unit inner strides, row
+ * strides in elements).
  * kind 1: g sigmoid(g) u;  kind 2: g' = min(g, limit), u' = clamp(u, -limit, limit), g' sigmoid(alpha g') (u' + 1). */
 #define GBXM_GLU_SILU 1
 #define GBXM_GLU_CLAMPED_SWISH 2
 #define GBXM_GLU_GELU_TANH 3      /* gelu(g) u, gelu in its tanh form */
 #define GBXM_GLU_SIGMOID 4        /* sigmoid(g) u */
-int gbxm_glu(const void* gu, int64_t gu_stride, void* out, int64_t T, int32_t F, int32_t kind, float limit, float alpha, int32_t act, void* stream);
+int gbxm_glu(const void* gu, int64_t gu_stride, const float* scale, int64_t scale_row, void* out, int64_t out_row, int64_t T, int32_t F, int32_t kind,
+             float limit, float alpha, int32_t act, void* stream);
 /* Router decisions from fp32 logits [T][E]: s = sigmoid(logit), choice score c = s + correction; with n_groups > 0 the experts form
  * n_groups equal groups of neighbours, a group's score is the sum of its two largest c, and only experts of the keep_groups best
  * groups can be chosen; the `top` largest c are chosen (ties: lower index); weight = s (divided by the chosen sum + 1e-20 if
@@ -197,9 +204,10 @@ int gbxm_conv_tail_update(const void* y, int64_t y_stride, void* tail, const int
  * S <- S + k u^T; o = S^T q.  T: rows of the step (chooses the workgroup shape).  dk <= 256. */
 int gbxm_state_scan(const float* r, int64_t r_stride, float* state, float* out, const int32_t* seq, int32_t B, int64_t T, int32_t H, int32_t G,
                     int32_t dk, int32_t dv, int32_t delta, void* stream);
-/* out[t][h][c] = o[t][h][c] / sqrt(mean_c o^2 + eps) * w[c] * gate(g[t][h][c]); gate kind 1 silu, 2 sigmoid; o fp32, g / out activation dtype. */
-int gbxm_head_norm_gate(const float* o, const void* gate, int64_t gate_stride, const float* w, void* out, int64_t T, int32_t H, int32_t dv,
-                        float eps, int32_t kind, int32_t act, void* stream);
+/* out[t][h][c] = o[t][h][c] / sqrt(mean_c o^2 + eps) * w[c] * gate(g[t][h][c]); gate kind 1 silu, 2 sigmoid; o fp32, g / out activation dtype;
+ * w null: no weight. */
+int gbxm_head_norm_gate(const float* o, const void* gate, int64_t gate_stride, const float* w, void* out, int64_t out_row, int64_t T, int32_t H,
+                        int32_t dv, float eps, int32_t kind, int32_t act, void* stream);
 
 /* ---- sandwich-norm layers, token shift, hashed pair embedding (gbx-lm_amd/models/residual.py, models/embedding.py) ---- */
 
@@ -238,6 +246,80 @@ int gbxm_block_gate_logits(const float* u, const void* w, const float* bias, flo
  * 0; written back); out[t][c] = S * gelu_tanh(y[t][c]) in the activation dtype. */
 int gbxm_gated_lru_scan(const float* u, const float* logits, int64_t lg_t, int64_t lg_b, const float* lam_sp, const void* y, int64_t y_stride, float* state, void* out,
                         const int32_t* seq, int32_t B, int64_t T, int32_t C, int32_t bs, float rate, int32_t act, void* stream);
+
+/* ---- recurrent mixers with one decay per head and token (gbx-lm_amd/models/recurrent_mixers.py) ---- */
+
+/* Rows of a state space mixer.  y rows hold C channels x | B | C at off_x and H step sizes at off_dt.
+ * out[t][c] = silu(bias[c] + sum_j conv[j][c] y[t - (taps-1) + j][off_x + c]) in the activation dtype (conv [taps][C]; inputs before the
+ * step from tail [slots][taps-1][C], oldest first; zeros before the sequence);  w = softplus(y[t][off_dt + h] + dt_bias[h]),
+ * dt_out[t] = (-rate[h] w for all h) | (w for all h), fp32.  move_tail (steps with one row per sequence only): the row's inputs also
+ * enter the tail; otherwise gbxm_conv_tail_update does that afterwards. */
+typedef struct {
+  const void* y;    int64_t y_stride;
+  const void* conv;
+  const float* bias;            /* [C] or null */
+  void* tail;
+  const float* dt_bias;         /* [H] */
+  const float* rate;            /* [H] */
+  const int32_t* seq;
+  const int32_t* tok;
+  void* out;                    /* [T][C] */
+  float* dt_out;                /* [T][2 H] */
+  int64_t T;
+  int32_t C, H, taps, off_x, off_dt, move_tail, act;
+} gbxm_ssm_prepare_args;
+int gbxm_ssm_prepare(const gbxm_ssm_prepare_args* a, void* stream);
+/* S <- d S + w k v^T,  o = scale S^T q + skip[h] v  per head h over each sequence's new rows; q, k [G][dk] and v [H][dv] at off_q / off_k /
+ * off_v of rows of the activation dtype (head h reads q / k group h / (H / G)); d = decay[h], or exp(log_decay[t * dt_stride + h]) when
+ * decay is null; w = write[t * dt_stride + h] or 1; skip may be null.  state fp32 [slots][H][dv][dk] (read unless the sequence starts at
+ * position 0, written back), out fp32 [T][H*dv].  T: rows of the step (chooses the kernel).  dk <= 256. */
+typedef struct {
+  const void* rows; int64_t row_stride;
+  const float* decay;
+  const float* log_decay;
+  const float* write; int64_t dt_stride;
+  const float* skip;
+  float* state;
+  float* out;
+  const int32_t* seq;
+  int64_t T;
+  int32_t B, H, G, dk, dv, off_q, off_k, off_v;
+  float scale;
+  int32_t act;
+} gbxm_head_scan_args;
+int gbxm_head_scan(const gbxm_head_scan_args* a, void* stream);
+/* v = o * silu(z); out = v / sqrt(mean of v^2 over its part + eps) * w, a row being `groups` parts of `size` channels.  o fp32 [T][n],
+ * w fp32 [n], z and out rows of the activation dtype. */
+int gbxm_gate_group_norm(const float* o, const void* z, int64_t z_stride, const float* w, void* out, int64_t out_stride, int64_t T, int32_t groups,
+                         int32_t size, float eps, int32_t act, void* stream);
+
+/* ---- parallel layers with routed experts (gbx-lm_amd/models/residual.py:layer_update_, models/switch_layers.py) ---- */
+
+/* v = (replace ? 0 : x[t]) + branch[t] + sum_{k < top} mix[t * mix_row + k] cand[t][k] + extra[t];  x[t] <- v;  image[t] = v in the activation
+ * dtype (row stride image_row);  h[t] = rms_norm(v) * norm_w in the activation dtype.  cand / extra / image / norm_w may be null;
+ * top <= 64. */
+typedef struct {
+  float* x;
+  const void* branch; int64_t branch_row;
+  const void* cand;
+  const float* mix; int64_t mix_row;
+  const void* extra;
+  const float* norm_w;
+  void* h;
+  void* image; int64_t image_row;
+  int64_t T;
+  int32_t width, top, replace;
+  float eps;
+  int32_t act;
+} gbxm_layer_update_args;
+int gbxm_layer_update(const gbxm_layer_update_args* a, void* stream);
+/* logits[t][e] = sum_k h[t][k] router[e][k] in fp32, for few rows. */
+int gbxm_router_rows(const void* h, const float* router, float* logits, int64_t T, int32_t K, int32_t E, int32_t act, void* stream);
+/* Router decisions from fp32 logit rows (stride `row`): s = softmax over E; with n_groups > 0 only experts of the keep_groups groups (equal
+ * groups of neighbours) with the largest s in them; the `top` largest s (ties: lower index), weights = s as they are.  gate: logit E of a
+ * row is a gate's, weight[top] = its sigmoid. */
+int gbxm_route_groups(const float* logits, int64_t row, int32_t* idx, float* weight, int64_t weight_row, int64_t T, int32_t E, int32_t top,
+                      int32_t n_groups, int32_t keep_groups, int32_t gate, void* stream);
 
 #ifdef __cplusplus
 }
