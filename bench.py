@@ -776,9 +776,89 @@ def laruzen_bench(args):
     print(json.dumps({"metric": "laruzen_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "sizes": out}))
 
 
+LERIPEL_SIZES = {
+    # name: Leripel geometry (r retention, m state space mixer, a chunked attention; routed experts with a gated shared one in every layer)
+    # and, from it, the Laruzen (the closest existing model: dense bf16 decoder over ragged steps with linear-attention states, attention
+    # and routed experts with a shared one) of equal width, layer runs and experts: lightning attention of the retention's geometry for r,
+    # gated linear attention with as many state columns for m, the attention's geometry in the pair for a
+    "small": dict(width=1024, retention=dict(heads=4, dim=128, vdim=256), mamba2=dict(heads=32, vdim=64, state=128, groups=1, conv=4, norm_groups=1),
+                  attention=dict(heads=16, kv_heads=4, dim=64, vdim=64, chunk=1024), moe=dict(experts=32, top=4, ff=512, groups=(8, 4), shared=1024),
+                  pattern="rmra"),
+    "a3b-like": dict(width=2048, retention=dict(heads=8, dim=128, vdim=256), mamba2=dict(heads=64, vdim=64, state=128, groups=8, conv=4, norm_groups=8),
+                     attention=dict(heads=16, kv_heads=4, dim=128, vdim=128, chunk=4096), moe=dict(experts=128, top=8, ff=768, groups=(8, 4), shared=1536),
+                     pattern="rmra"),
+    "looped": dict(width=2048, retention=dict(heads=8, dim=128, vdim=256), mamba2=dict(heads=64, vdim=64, state=128, groups=1, conv=4, norm_groups=1),
+                   attention=dict(heads=16, kv_heads=2, dim=128, vdim=128, chunk=2048), moe=dict(experts=64, top=4, ff=1024, groups=(4, 2), shared=1024),
+                   pattern="mra", loop=(0, 2, 2)),
+}
+
+
+def leripel_bench(args):
+    """``--design leripel``: prefill and decode throughput of Leripel at layer sizes of real models (random weights, bf16), beside
+    Laruzen of equal width, layer runs, routed experts and state geometry.  One JSON line; the default workload of
+    this file is untouched."""
+    from gbx_lm_amd import synthetic as S
+    from gbx_lm_amd.batching import BatchScheduler
+    dev = torch.device("cuda", 0)
+    torch.cuda.set_device(dev)
+
+    def clock(fn, reps):
+        fn()
+        fn()                                         # (the second call of a shape still pays one-time allocations)
+        torch.cuda.synchronize()
+        e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+        e0.record()
+        for _ in range(reps):
+            fn()
+        e1.record()
+        torch.cuda.synchronize()
+        return e0.elapsed_time(e1) / reps
+
+    def legs(model, vocab, tag, res):
+        toks = lambda n, o=0: [(o + i * 7919) % vocab for i in range(n)]
+        for T in (512, 4096):
+            def prefill():
+                eng = BatchScheduler(model)
+                eng.step([("p", toks(T))])
+            res[f"{tag}prefill_T{T}_tok_s"] = round(T / clock(prefill, 3) * 1e3)
+        for B, ctx in ((1, 2048), (32, 256)):
+            eng = BatchScheduler(model)
+            eng.step([(i, toks(ctx, i)) for i in range(B)])
+            state = {"t": 0}
+            def decode():
+                state["t"] += 1
+                eng.step([(i, [(state["t"] * 31 + i) % vocab]) for i in range(B)])
+            res[f"{tag}decode_B{B}_ctx{ctx}_tok_s"] = round(B / clock(decode, 64) * 1e3)
+            del eng
+        print(tag or "leripel", res, file=sys.stderr, flush=True)
+
+    out = {}
+    for name in args.sizes.split(","):
+        g = LERIPEL_SIZES[name]
+        res = {"geometry": g}
+        cfg = S.leripel_config(**g)
+        model = S.build_leripel(cfg, device=dev, seed=0)
+        legs(model, cfg["vocab"], "", res)
+        runs = [cfg["layers"][i]["type"] for i in model.layer_runs]
+        del model
+        torch.cuda.empty_cache()
+        r, m, a, e = g["retention"], g["mamba2"], g["attention"], g["moe"]
+        lm = S.build_laruzen(S.laruzen_config(width=g["width"], gla=dict(heads=m["heads"] * m["vdim"] // 256, dim=m["state"], vdim=256, tau=16.0), lightning=r,
+                                              left=dict(heads=a["heads"], kv_heads=a["kv_heads"], dim=a["dim"], vdim=a["vdim"], window=a["chunk"]),
+                                              right=dict(width=g["width"], blocks=8, conv=4), ff=e["top"] * e["ff"] + e["shared"],
+                                              moe=dict(experts=e["experts"], top=e["top"], ff=e["ff"], shared=e["shared"]),
+                                              pattern="".join({"retention": "l", "mamba2": "g", "attention": "p"}[k] for k in runs), vocab=cfg["vocab"]),
+                             device=dev, seed=0)
+        legs(lm, cfg["vocab"], "laruzen_", res)
+        del lm
+        torch.cuda.empty_cache()
+        out[name] = res
+    print(json.dumps({"metric": "leripel_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "sizes": out}))
+
+
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", default=None, choices=["revitar", "radenex", "tugolix", "laruzen"], help="side benchmark of one model design beside the closest existing "
+    ap.add_argument("--design", default=None, choices=["revitar", "radenex", "tugolix", "laruzen", "leripel"], help="side benchmark of one model design beside the closest existing "
                     "family at equal size (own JSON line; the default workload and its output are unchanged)")
     ap.add_argument("--sizes", default=None, help="--design: comma-separated names of REVITAR_SIZES (default small,a3b-like) / RADENEX_SIZES "
                     "(default small,lite-like) / TUGOLIX_SIZES (default small,a3b-like)")
@@ -800,8 +880,9 @@ def main():
     if args.design is not None:
         if not torch.cuda.is_available():
             raise SystemExit("bench.py needs an MI355X")
-        args.sizes = args.sizes or {"revitar": "small,a3b-like", "radenex": "small,lite-like", "tugolix": "small,a3b-like", "laruzen": "small,a3b-like"}[args.design]
-        return {"revitar": revitar_bench, "radenex": radenex_bench, "tugolix": tugolix_bench, "laruzen": laruzen_bench}[args.design](args)
+        args.sizes = args.sizes or {"revitar": "small,a3b-like", "radenex": "small,lite-like", "tugolix": "small,a3b-like", "laruzen": "small,a3b-like", "leripel": "small,a3b-like"}[args.design]
+        return {"revitar": revitar_bench, "radenex": radenex_bench, "tugolix": tugolix_bench, "laruzen": laruzen_bench,
+                "leripel": leripel_bench}[args.design](args)
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:
         spawn_ranks(args.gpus)                                     # never returns; nothing has touched the GPU yet
     world = int(os.environ.get("WORLD_SIZE", "1"))

@@ -577,3 +577,95 @@ def build_laruzen(config: Dict, device="cpu", seed: int = 0, act_dtype=torch.bfl
         raise ValueError(f"tensors without a place in the model: {skipped[:3]}")
     model.eval()
     return model
+
+
+# ------------------------------------------------------------------------------------------------ Leripel (parallel layers; retention, state space and chunked attention mixers)
+def leripel_config(width: int, retention: Dict, mamba2: Dict, attention: Dict, moe: Dict, pattern: str = "rmra", loop=None, vocab: int = 32000) -> Dict:
+    """config.json of a Leripel model: ``pattern`` names the layers in order ('r' retention, 'm' state space, 'a' chunked attention).
+    ``retention``: heads, dim, vdim (decays spread over the heads); ``mamba2``: heads, vdim, state, groups, conv, norm_groups;
+    ``attention``: heads, kv_heads, dim, vdim, chunk, rot_dims; ``moe``: experts, top, ff, groups (count, keep) or None, shared or None;
+    ``loop``: (start, stop, times) or None."""
+    router = {"experts": moe["experts"], "top": moe["top"]}
+    if moe.get("groups"):
+        router["groups"] = {"count": moe["groups"][0], "keep": moe["groups"][1]}
+    routed = {"kind": "moe", "expert": {"ff": moe["ff"]}, "router": router, "shared": {"ff": moe["shared"]} if moe.get("shared") else None}
+    layers = []
+    for c in pattern:
+        if c == "r":
+            h = retention["heads"]
+            layer = {"type": "retention", "mixer": dict({k: retention[k] for k in ("heads", "dim", "vdim")}, decay=[1.0 - 2.0 ** (-5 - 7.0 * j / max(h - 1, 1)) for j in range(h)])}
+        elif c == "m":
+            layer = {"type": "mamba2", "mixer": {k: mamba2[k] for k in ("heads", "vdim", "state", "groups", "conv", "norm_groups")}}
+        elif c == "a":
+            layer = {"type": "attention", "mixer": {"heads": attention["heads"], "kv_heads": attention["kv_heads"], "dim": attention["dim"], "vdim": attention["vdim"],
+                                                    "scale": attention["dim"] ** -0.5, "mask": {"size": attention["chunk"]},
+                                                    "rot": {"base": 1e6, "dims": attention.get("rot_dims", attention["dim"])}}}
+        else:
+            raise ValueError(f"leripel_config: unknown layer letter {c!r}")
+        layers.append(dict(layer, mlp=json.loads(json.dumps(routed))))
+    return {"architecture": "Leripel", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": layers,
+            "loop": None if loop is None else {"start": loop[0], "stop": loop[1], "times": loop[2]}}
+
+
+def leripel_checkpoint(config: Dict, device="cpu", seed: int = 0, dtype=torch.bfloat16) -> Dict[str, torch.Tensor]:
+    """Random tensors in the design's checkpoint names with real shapes, generated directly on ``device``."""
+    device = torch.device(device)
+    gen = torch.Generator(device=device)
+    gen.manual_seed(seed)
+    W = config["width"]
+
+    def mat(o, i, mult=1.0):
+        return (torch.randn((o, i), device=device, generator=gen) * (mult * i ** -0.5)).to(dtype)
+
+    def vec(n, lo, hi):
+        return (torch.rand((n,), device=device, generator=gen) * (hi - lo) + lo).to(dtype)
+
+    w = {"embed": torch.randn((config["vocab"], W), device=device, generator=gen).to(dtype), "final.norm": vec(W, 0.9, 1.1), "head": mat(config["vocab"], W)}
+    if config.get("loop"):
+        w["loop.in"] = mat(W, 2 * W)
+    for i, layer in enumerate(config["layers"]):
+        p, m, kind = f"l{i}.", layer["mixer"], layer["type"]
+        w[p + "norm1"] = vec(W, 0.9, 1.1)
+        x, H, dv = p + "mix.", m["heads"], m["vdim"]
+        w[x + "o"] = mat(W, H * dv)
+        if kind == "mamba2":
+            inner, gn = H * dv, m["groups"] * m["state"]
+            w[x + "in"] = mat(2 * inner + 2 * gn + H, W)
+            w[x + "conv"], w[x + "conv.b"] = (torch.randn((inner + 2 * gn, m["conv"]), device=device, generator=gen) * 0.5 + 0.25).to(dtype), vec(inner + 2 * gn, -0.1, 0.1)
+            w[x + "dt_bias"], w[x + "A_log"], w[x + "D"], w[x + "norm"] = vec(H, -4.0, -1.0), vec(H, 0.0, 2.0), vec(H, 0.5, 1.0), vec(inner, 0.9, 1.1)
+        else:
+            G, d = m.get("kv_heads", H), m["dim"]
+            w[x + "q"], w[x + "k"], w[x + "v"] = mat(H * d, W), mat(G * d, W), mat(G * dv, W)
+            w[x + "g"] = mat(H if kind == "attention" else H * dv, W)
+            if kind == "attention":
+                w[x + "temp"] = vec(H, 0.9, 1.1)
+        ff = layer.get("mlp")
+        if ff is not None:
+            f, n, E = p + "mlp.", ff["expert"]["ff"], ff["router"]["experts"]
+            w[f + "router"] = mat(E, W, 2.0)
+            for e in range(E):
+                w[f + f"e{e}.gate"], w[f + f"e{e}.up"], w[f + f"e{e}.down"] = mat(n, W), mat(n, W), mat(W, n)
+            if ff.get("shared"):
+                s = ff["shared"]["ff"]
+                w[f + "shared.gate"], w[f + "shared.up"], w[f + "shared.down"], w[f + "shared.sg"] = mat(s, W), mat(s, W), mat(W, s), mat(1, W)
+    return w
+
+
+def build_leripel(config: Dict, device="cpu", seed: int = 0, act_dtype=torch.bfloat16):
+    """Random-init Leripel with real shapes: a random checkpoint generated on ``device`` goes through the model's own ``sanitize``."""
+    from .models import leripel
+    from .utils import load_weights
+    device = torch.device(device)
+    weights = leripel_checkpoint(config, device, seed)
+    args = leripel.ModelArgs.from_dict(config)
+    model = leripel.Model(args)                   # (the buffers the constructors compute -- decays, frequency tables -- are tiny)
+    weights = model.sanitize(weights)
+    weights = {k: (v.to(act_dtype) if v.is_floating_point() and v.dtype != torch.float32 else v) for k, v in weights.items()}
+    with torch.device("meta"):
+        model = leripel.Model(args)
+    model = model.to_empty(device=device)
+    skipped = load_weights(model, weights, device=device)
+    if skipped:
+        raise ValueError(f"tensors without a place in the model: {skipped[:3]}")
+    model.eval()
+    return model
