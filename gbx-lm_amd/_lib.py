@@ -357,7 +357,8 @@ class HeadScanArgs(ctypes.Structure):
                 ("write", ctypes.c_void_p), ("dt_stride", ctypes.c_int64), ("skip", ctypes.c_void_p), ("state", ctypes.c_void_p), ("out", ctypes.c_void_p),
                 ("seq", ctypes.c_void_p), ("T", ctypes.c_int64), ("B", ctypes.c_int32), ("H", ctypes.c_int32), ("G", ctypes.c_int32), ("dk", ctypes.c_int32),
                 ("dv", ctypes.c_int32), ("off_q", ctypes.c_int32), ("off_k", ctypes.c_int32), ("off_v", ctypes.c_int32), ("scale", ctypes.c_float),
-                ("act", ctypes.c_int32)]
+                ("act", ctypes.c_int32), ("tiles", ctypes.c_void_p), ("n_tiles", ctypes.c_int64), ("q_tile", ctypes.c_int32), ("ws", ctypes.c_void_p),
+                ("ws_bytes", ctypes.c_size_t)]
 
 
 class LayerUpdateArgs(ctypes.Structure):
@@ -430,6 +431,8 @@ def mixers() -> ctypes.CDLL:
         L.gbxm_block_gate_logits.argtypes = [p, p, p, p, i64, i32, i32, i32, i32, p]
         L.gbxm_gated_lru_scan.argtypes = [p, p, i64, i64, p, p, i64, p, p, p, i32, i64, i32, i32, f32, i32, p]
         L.gbxm_ssm_prepare.argtypes = [ctypes.POINTER(SsmPrepareArgs), p]
+        L.gbxm_head_scan_workspace.argtypes = [i64, i32, i64, i32, i32, i32, i32, i32]
+        L.gbxm_head_scan_workspace.restype = sz
         L.gbxm_head_scan.argtypes = [ctypes.POINTER(HeadScanArgs), p]
         L.gbxm_gate_group_norm.argtypes = [p, p, i64, p, p, i64, i64, i32, i32, f32, i32, p]
         L.gbxm_layer_update.argtypes = [ctypes.POINTER(LayerUpdateArgs), p]

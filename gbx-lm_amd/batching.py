@@ -157,6 +157,8 @@ class BatchScheduler:
                     raise ValueError("a wanted place lies outside the entry's tokens")
                 if not rows:
                     return torch.empty((0, self.model.args.vocab), dtype=torch.float32, device=self.device)
+                if len(rows) == len(slot):
+                    return logits.float() if logits.dtype != torch.float32 else logits.clone()      # (the graph's buffer is overwritten by the next replay)
                 return logits.index_select(0, torch.tensor(rows, dtype=torch.long, device=self.device)).float()
         batch = StepBatch.build(slot, pos0, n_new, self.device)
         tokens = torch.tensor([t for _, ts in entries for t in ts], dtype=torch.long)

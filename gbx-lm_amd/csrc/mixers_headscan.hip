@@ -9,6 +9,7 @@
 //                           holds R x 4 neighbouring key channels; operands straight from the rows.  Bound by the state's traffic.
 //   head_scan_kernel<R>     longer portions: the same arithmetic with the operands of a chunk of tokens in LDS, shared by 16 columns, the
 //                           next chunk fetched while the current one is computed.
+//                           (bf16 prompt portions on the 16-byte grid: chunk kernels on the matrix cores, mixers_headscan_mfma.hip)
 //   gate_group_norm_kernel  v = o * silu(z), each of the equal parts of a row scaled by its own root mean square, times a weight.
 //
 // q, k, v are read from rows of the activation dtype (a projection's rows, or the prepared ones); decays, write factors, the state and
@@ -323,6 +324,11 @@ bool act_ok(int act) { return act == GBXM_BF16 || act == GBXM_F32; }
 bool aligned(const void* p, size_t n) { return reinterpret_cast<uintptr_t>(p) % n == 0; }
 
 }  // namespace
+
+bool head_chunks_shape(const gbxm_head_scan_args& a);                       // mixers_headscan_mfma.hip
+int launch_head_chunks(const gbxm_head_scan_args& a, hipStream_t s);
+size_t head_chunks_workspace(int64_t n_tiles, int H, int dk, int dv);
+
 }  // namespace gbxm
 
 using namespace gbxm;
@@ -352,6 +358,11 @@ int gbxm_ssm_prepare(const gbxm_ssm_prepare_args* a, void* stream) {
   return after_launch("ssm_prepare");
 }
 
+size_t gbxm_head_scan_workspace(int64_t T_, int32_t B, int64_t n_tiles, int32_t q_tile, int32_t H, int32_t dk, int32_t dv, int32_t act) {
+  if (act != GBXM_BF16 || q_tile != 128 || n_tiles < 1 || T_ < 32 * static_cast<int64_t>(B) || dk % 8 || dv % 8 || dk > 256) return 0;
+  return head_chunks_workspace(n_tiles, H, dk, dv);
+}
+
 int gbxm_head_scan(const gbxm_head_scan_args* a, void* stream) {
   if (!a || !act_ok(a->act) || !a->rows || !a->state || !a->out || !a->seq || a->B < 0 || a->T < 0 || a->H < 1 || a->G < 1 || a->H % a->G || a->dk < 1 ||
       a->dv < 1 || (!a->decay && !a->log_decay) || ((a->log_decay || a->write) && a->dt_stride < a->H) || a->off_q < 0 || a->off_k < 0 || a->off_v < 0 ||
@@ -363,6 +374,7 @@ int gbxm_head_scan(const gbxm_head_scan_args* a, void* stream) {
   if (a->B > 65535 || a->H > 65535) return fail(GBXM_ERR_UNSUPPORTED, "head_scan: grid");
   hipStream_t s = static_cast<hipStream_t>(stream);
   const bool bf = a->act == GBXM_BF16;
+  if (head_chunks_shape(*a)) return launch_head_chunks(*a, s);
   if (a->T >= 8 * static_cast<int64_t>(a->B)) return bf ? launch_scan<bf16_t>(*a, s) : launch_scan<float>(*a, s);
   const size_t vb = bf ? 8 : 16;
   const bool vec = a->dk % 4 == 0 && a->row_stride % 4 == 0 && a->off_q % 4 == 0 && a->off_k % 4 == 0 && aligned(a->rows, vb) && aligned(a->state, 16);

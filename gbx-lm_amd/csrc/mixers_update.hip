@@ -116,66 +116,74 @@ __global__ __launch_bounds__(NT) void router_rows_kernel(const T* __restrict__ h
   if (lane == 0) logits[t * E + e] = s;
 }
 
-// One wave per row.  LDS: logits of the experts (the choice runs on them: softmax keeps their order), then group maxima.
-__global__ __launch_bounds__(64) void route_groups_kernel(const float* __restrict__ logits, int64_t row, int* __restrict__ idx, float* __restrict__ weight,
+// One workgroup per row.  The choice runs on the logits (softmax keeps their order) and by RANK: an expert counts the candidates in front
+// of it -- larger, or equal with a lower index -- so no round waits for another; ranks are a permutation (a logit that is not a number
+// counts as the smallest).  LDS: candidate logits [E, padded to 4 with -inf], group maxima [n_groups, padded], partial sums.
+__global__ __launch_bounds__(NT) void route_groups_kernel(const float* __restrict__ logits, int64_t row, int* __restrict__ idx, float* __restrict__ weight,
                                                          int64_t weight_row, int E, int top, int n_groups, int keep_groups, int gate) {
-  extern __shared__ float lds[];
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  __shared__ float red[NW];
   float* cl = lds;
-  float* gl = lds + E;
+  float* gl = lds + (E + 3) / 4 * 4;
   const int64_t t = blockIdx.x;
-  const int lane = threadIdx.x;
+  const int nth = blockDim.x, tid = threadIdx.x;
   const float* lr = logits + t * row;
+  auto at = [&](int e) { const float v = lr[e]; return v == v ? v : -INFINITY; };
+  for (int e = tid; e < (E + 3) / 4 * 4; e += nth) cl[e] = e < E ? at(e) : -INFINITY;
+  __syncthreads();
+  auto rank_of = [&](const float* v, int n4, int e, float x) {
+    int rank = 0;
+    for (int j = 0; j < n4; ++j) {
+      const float4 u = *reinterpret_cast<const float4*>(v + 4 * j);
+      const float w[4] = {u.x, u.y, u.z, u.w};
+#pragma unroll
+      for (int k = 0; k < 4; ++k) rank += (w[k] > x || (w[k] == x && 4 * j + k < e)) ? 1 : 0;
+    }
+    return rank;
+  };
   float mx = -INFINITY;
-  for (int e = lane; e < E; e += 64) { cl[e] = lr[e]; mx = fmaxf(mx, lr[e]); }
+  for (int e = tid; e < E; e += nth) mx = fmaxf(mx, cl[e]);
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o, 64));
+  if (nth > 64) {
+    if ((tid & 63) == 0) red[tid >> 6] = mx;
+    __syncthreads();
+    for (int i = 0; i < nth / 64; ++i) mx = fmaxf(mx, red[i]);
+    __syncthreads();
+  }
   float sum = 0.f;
-  for (int e = lane; e < E; e += 64) sum += expf(lr[e] - mx);
+  for (int e = tid; e < E; e += nth) sum += expf(cl[e] - mx);
   sum = wave_sum(sum);
-  __syncthreads();
-  // arg-max over n values (ties: the lower index); every lane gets the result
-  auto arg_max = [&](const float* v, int n) {
-    float bv = -INFINITY;
-    int bi = 0x7fffffff;
-    for (int e = lane; e < n; e += 64)
-      if (v[e] > bv || bi == 0x7fffffff) { bv = v[e]; bi = e; }
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float ov = __shfl_xor(bv, o, 64);
-      const int oi = __shfl_xor(bi, o, 64);
-      if (oi != 0x7fffffff && (bi == 0x7fffffff || ov > bv || (ov == bv && oi < bi))) { bv = ov; bi = oi; }
-    }
-    return bi;
-  };
+  if (nth > 64) {
+    if ((tid & 63) == 0) red[tid >> 6] = sum;
+    __syncthreads();
+    sum = 0.f;
+    for (int i = 0; i < nth / 64; ++i) sum += red[i];
+  }
   if (n_groups > 0) {
-    const int size = E / n_groups;
-    for (int g = lane; g < n_groups; g += 64) {
+    const int size = E / n_groups, g4 = (n_groups + 3) / 4;
+    for (int g = tid; g < 4 * g4; g += nth) {
       float a = -INFINITY;
-      for (int e = g * size; e < (g + 1) * size; ++e) a = fmaxf(a, cl[e]);
+      if (g < n_groups)
+        for (int e = g * size; e < (g + 1) * size; ++e) a = fmaxf(a, cl[e]);
       gl[g] = a;
     }
     __syncthreads();
-    for (int k = 0; k < keep_groups; ++k) {
-      const int g = arg_max(gl, n_groups);
-      __syncthreads();
-      if (lane == 0) gl[g] = -INFINITY;            // taken: -inf marks a kept group from here on (logits are finite)
-      __syncthreads();
-    }
-    for (int e = lane; e < E; e += 64)
-      if (gl[e / size] != -INFINITY) cl[e] = -INFINITY;
-    __syncthreads();
-  }
-  for (int k = 0; k < top; ++k) {
-    const int e = arg_max(cl, E);
-    __syncthreads();
-    if (lane == 0) {
-      idx[t * top + k] = e;
-      weight[t * weight_row + k] = expf(lr[e] - mx) / sum;
-      cl[e] = -INFINITY;
+    for (int e = tid; e < E; e += nth) {
+      const int g = e / size;
+      if (rank_of(gl, g4, g, gl[g]) >= keep_groups) cl[e] = -INFINITY;      // (only this thread reads cl[e] until the barrier)
     }
     __syncthreads();
   }
-  if (gate && lane == 0) weight[t * weight_row + top] = 1.f / (1.f + expf(-lr[E]));
+  for (int e = tid; e < E; e += nth) {
+    const float x = cl[e];
+    const int rank = rank_of(cl, (E + 3) / 4, e, x);
+    if (rank < top) {
+      idx[t * top + rank] = e;
+      weight[t * weight_row + rank] = expf(x - mx) / sum;
+    }
+  }
+  if (gate && tid == 0) weight[t * weight_row + top] = 1.f / (1.f + expf(-lr[E]));
 }
 
 bool act_ok(int act) { return act == GBXM_BF16 || act == GBXM_F32; }
@@ -234,8 +242,8 @@ int gbxm_route_groups(const float* logits, int64_t row, int32_t* idx, float* wei
   if (E > 8192) return fail(GBXM_ERR_UNSUPPORTED, "route_groups: more than 8192 experts");
   if (T_ == 0) return GBXM_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  route_groups_kernel<<<dim3(T_), 64, (E + (n_groups > 0 ? n_groups : 1)) * sizeof(float), s>>>(logits, row, idx, weight, weight_row, E, top, n_groups,
-                                                                                               keep_groups, gate);
+  const size_t lds = ((E + 3) / 4 * 4 + (n_groups + 3) / 4 * 4 + 4) * sizeof(float);
+  route_groups_kernel<<<dim3(T_), E <= 64 ? 64 : (E <= 128 ? 128 : NT), lds, s>>>(logits, row, idx, weight, weight_row, E, top, n_groups, keep_groups, gate);
   return after_launch("route_groups");
 }
 

@@ -632,6 +632,11 @@ def head_state_scan(rows: torch.Tensor, heads: int, groups: int, dk: int, dv: in
     a.skip = None if skip is None else _f32(skip, "skip").data_ptr()
     a.state, a.out, a.seq, a.T, a.B = state.data_ptr(), out.data_ptr(), batch.seq.data_ptr(), t, len(batch.slot)
     a.H, a.G, a.dk, a.dv, a.off_q, a.off_k, a.off_v, a.scale, a.act = heads, groups, dk, dv, off_q, off_k, off_v, float(scale), act
+    if batch.tiles is not None and not batch.decode_only:
+        nbytes = _lib.mixers().gbxm_head_scan_workspace(t, a.B, batch.tiles.shape[0], batch.q_tile, heads, dk, dv, act)
+        if nbytes:
+            ws = torch.empty((nbytes,), dtype=torch.uint8, device=rows.device)
+            a.tiles, a.n_tiles, a.q_tile, a.ws, a.ws_bytes = batch.tiles.data_ptr(), batch.tiles.shape[0], batch.q_tile, ws.data_ptr(), nbytes
     _lib.check_mixers(_lib.mixers().gbxm_head_scan(ctypes.byref(a), _stream(rows.device)))
     return out
 

@@ -272,7 +272,8 @@ int gbxm_ssm_prepare(const gbxm_ssm_prepare_args* a, void* stream);
 /* S <- d S + w k v^T,  o = scale S^T q + skip[h] v  per head h over each sequence's new rows; q, k [G][dk] and v [H][dv] at off_q / off_k /
  * off_v of rows of the activation dtype (head h reads q / k group h / (H / G)); d = decay[h], or exp(log_decay[t * dt_stride + h]) when
  * decay is null; w = write[t * dt_stride + h] or 1; skip may be null.  state fp32 [slots][H][dv][dk] (read unless the sequence starts at
- * position 0, written back), out fp32 [T][H*dv].  T: rows of the step (chooses the kernel).  dk <= 256. */
+ * position 0, written back), out fp32 [T][H*dv].  T: rows of the step (chooses the kernel).  dk <= 256.  With a workspace of
+ * gbxm_head_scan_workspace bytes (0: not a step for it) and the step's tile table, bf16 prompt portions run in chunks on the matrix cores. */
 typedef struct {
   const void* rows; int64_t row_stride;
   const float* decay;
@@ -286,7 +287,12 @@ typedef struct {
   int32_t B, H, G, dk, dv, off_q, off_k, off_v;
   float scale;
   int32_t act;
+  const int32_t* tiles;         /* [n_tiles][2] */
+  int64_t n_tiles;
+  int32_t q_tile;
+  void* ws; size_t ws_bytes;
 } gbxm_head_scan_args;
+size_t gbxm_head_scan_workspace(int64_t T, int32_t B, int64_t n_tiles, int32_t q_tile, int32_t H, int32_t dk, int32_t dv, int32_t act);
 int gbxm_head_scan(const gbxm_head_scan_args* a, void* stream);
 /* v = o * silu(z); out = v / sqrt(mean of v^2 over its part + eps) * w, a row being `groups` parts of `size` channels.  o fp32 [T][n],
  * w fp32 [n], z and out rows of the activation dtype. */

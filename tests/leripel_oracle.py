@@ -228,8 +228,10 @@ def make_config(layers, vocab=61, width=64, eps=1e-5, loop=None):
             "loop": None if loop is None else {"start": loop[0], "stop": loop[1], "times": loop[2]}}
 
 
-def make_weights(cfg, seed=0, wide_router=False):
-    """``wide_router``: router rows are large and far apart, so that the rounding of a token's input rarely changes its experts."""
+def make_weights(cfg, seed=0, steady=False):
+    """``steady``: a retention head's keys lie near its queries.  A sequence's first read-out is <q, k> v / sqrt(dk) before its norm: with
+    unrelated q and k the product is near zero now and then, and the norm turns its rounding into a change of sign.  Output projections
+    are halved, so that a row's rounding is not amplified run after run."""
     gen = torch.Generator().manual_seed(seed)
     W = cfg["width"]
     bf = torch.bfloat16
@@ -251,6 +253,8 @@ def make_weights(cfg, seed=0, wide_router=False):
         if kind == "retention":
             d = m["dim"]
             w[x + "q"], w[x + "k"], w[x + "v"], w[x + "g"], w[x + "o"] = mat(H * d, W), mat(H * d, W), mat(H * dv, W), mat(H * dv, W), mat(W, H * dv)
+            if steady:
+                w[x + "k"] = (w[x + "q"].float() + 0.5 * w[x + "k"].float()).to(bf)
         elif kind == "mamba2":
             inner, gn = H * dv, m["groups"] * m["state"]
             w[x + "in"] = mat(2 * inner + 2 * gn + H, W)
@@ -262,10 +266,12 @@ def make_weights(cfg, seed=0, wide_router=False):
             G, d = m["kv_heads"], m["dim"]
             w[x + "q"], w[x + "k"], w[x + "v"], w[x + "g"], w[x + "o"] = mat(H * d, W), mat(G * d, W), mat(G * dv, W), mat(H, W, 2.0), mat(W, H * dv)
             w[x + "temp"] = vec(H, 0.5, 2.0)
+        if steady:
+            w[x + "o"] = 0.5 * w[x + "o"]
         ff = layer.get("mlp")
         if ff is not None:
             f, n, E = p + "mlp.", ff["expert"]["ff"], ff["router"]["experts"]
-            w[f + "router"] = mat(E, W, 6.0 if wide_router else 1.5)
+            w[f + "router"] = mat(E, W, 1.5)
             for e in range(E):
                 w[f + f"e{e}.gate"], w[f + f"e{e}.up"], w[f + f"e{e}.down"] = mat(n, W, 1.5), mat(n, W, 1.5), mat(W, n)
             if ff.get("shared"):
