@@ -154,7 +154,7 @@ __global__ __launch_bounds__(64 * NW) void head_step_kernel(gbxm_head_scan_args 
 // and write factors beside them.  Two buffers: a chunk is fetched into registers before the current one is computed.
 template <typename T, int R>
 __global__ __launch_bounds__(NT) void head_scan_kernel(gbxm_head_scan_args p) {
-  constexpr int DKP = 64 * R, NCOL = 16, ROW = 2 * DKP + NCOL, CH = R <= 1 ? 32 : (R <= 2 ? 16 : 8);
+  constexpr int DKP = 64 * R, NCOL = 16, ROW = 2 * DKP + NCOL, CH = R <= 1 ? 32 : (R <= 2 ? 16 : (R <= 4 ? 8 : 4));
   constexpr int PF = (CH * ROW + NT - 1) / NT;
   __shared__ __attribute__((aligned(16))) float buf[2][CH * ROW];
   __shared__ float dl[2][CH], wl[2][CH];
@@ -261,7 +261,8 @@ int launch_step(const gbxm_head_scan_args& a, bool vec, hipStream_t s) {
   } while (0)
   if (R <= 1) GBXM_STEP(1);
   else if (R <= 2) GBXM_STEP(2);
-  else GBXM_STEP(4);
+  else if (R <= 4) GBXM_STEP(4);
+  else GBXM_STEP(8);
 #undef GBXM_STEP
   return after_launch("head_scan (few rows)");
 }
@@ -272,7 +273,8 @@ int launch_scan(const gbxm_head_scan_args& a, hipStream_t s) {
   const int R = (a.dk + 63) / 64;
   if (R <= 1) head_scan_kernel<T, 1><<<grid, NT, 0, s>>>(a);
   else if (R <= 2) head_scan_kernel<T, 2><<<grid, NT, 0, s>>>(a);
-  else head_scan_kernel<T, 4><<<grid, NT, 0, s>>>(a);
+  else if (R <= 4) head_scan_kernel<T, 4><<<grid, NT, 0, s>>>(a);
+  else head_scan_kernel<T, 8><<<grid, NT, 0, s>>>(a);
   return after_launch("head_scan");
 }
 
@@ -369,7 +371,7 @@ int gbxm_head_scan(const gbxm_head_scan_args* a, void* stream) {
       a->off_q + static_cast<int64_t>(a->G) * a->dk > a->row_stride || a->off_k + static_cast<int64_t>(a->G) * a->dk > a->row_stride ||
       a->off_v + static_cast<int64_t>(a->H) * a->dv > a->row_stride)
     return fail(GBXM_ERR_INVALID, "head_scan: bad argument");
-  if (a->dk > 256) return fail(GBXM_ERR_UNSUPPORTED, "head_scan: %d key channels per head (at most 256)", a->dk);
+  if (a->dk > 512) return fail(GBXM_ERR_UNSUPPORTED, "head_scan: %d key channels per head (at most 512)", a->dk);
   if (a->B == 0 || a->T == 0) return GBXM_OK;
   if (a->B > 65535 || a->H > 65535) return fail(GBXM_ERR_UNSUPPORTED, "head_scan: grid");
   hipStream_t s = static_cast<hipStream_t>(stream);

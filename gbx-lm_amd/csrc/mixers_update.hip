@@ -133,6 +133,7 @@ __global__ __launch_bounds__(NT) void route_groups_kernel(const float* __restric
   __syncthreads();
   auto rank_of = [&](const float* v, int n4, int e, float x) {
     int rank = 0;
+#pragma unroll 8
     for (int j = 0; j < n4; ++j) {
       const float4 u = *reinterpret_cast<const float4*>(v + 4 * j);
       const float w[4] = {u.x, u.y, u.z, u.w};
@@ -165,6 +166,7 @@ __global__ __launch_bounds__(NT) void route_groups_kernel(const float* __restric
     for (int g = tid; g < 4 * g4; g += nth) {
       float a = -INFINITY;
       if (g < n_groups)
+#pragma unroll 8
         for (int e = g * size; e < (g + 1) * size; ++e) a = fmaxf(a, cl[e]);
       gl[g] = a;
     }

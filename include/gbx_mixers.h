@@ -272,7 +272,7 @@ int gbxm_ssm_prepare(const gbxm_ssm_prepare_args* a, void* stream);
 /* S <- d S + w k v^T,  o = scale S^T q + skip[h] v  per head h over each sequence's new rows; q, k [G][dk] and v [H][dv] at off_q / off_k /
  * off_v of rows of the activation dtype (head h reads q / k group h / (H / G)); d = decay[h], or exp(log_decay[t * dt_stride + h]) when
  * decay is null; w = write[t * dt_stride + h] or 1; skip may be null.  state fp32 [slots][H][dv][dk] (read unless the sequence starts at
- * position 0, written back), out fp32 [T][H*dv].  T: rows of the step (chooses the kernel).  dk <= 256.  With a workspace of
+ * position 0, written back), out fp32 [T][H*dv].  T: rows of the step (chooses the kernel).  dk <= 512.  With a workspace of
  * gbxm_head_scan_workspace bytes (0: not a step for it) and the step's tile table, bf16 prompt portions run in chunks on the matrix cores. */
 typedef struct {
   const void* rows; int64_t row_stride;

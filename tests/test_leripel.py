@@ -176,7 +176,7 @@ def test_mixers_alone(device, dtype, layer):
 
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("dk,dv,heads,groups", [(64, 64, 4, 2), (128, 128, 2, 2), (40, 72, 6, 1), (256, 24, 1, 1), (16, 8, 3, 3), (30, 9, 2, 1)])
+@pytest.mark.parametrize("dk,dv,heads,groups", [(64, 64, 4, 2), (128, 128, 2, 2), (40, 72, 6, 1), (256, 24, 1, 1), (400, 16, 2, 1), (16, 8, 3, 3), (30, 9, 2, 1)])
 def test_state_scan_is_32_bit(device, dtype, dk, dv, heads, groups):
     """The state, the decays and the sums are 32-bit in both dtypes and in every kernel form (q, k and v are the same bf16 numbers here):
     unequal sequences of one step with history, log decays per row from tiny to -40, write factors, skip.  Then one more step."""
