@@ -16,7 +16,7 @@ from typing import Callable, Dict, Iterable, List, Optional, Sequence, Tuple
 
 import torch
 
-from . import env
+from . import env, graphs
 
 
 @dataclass
@@ -97,7 +97,7 @@ class _DecodeGraph:
         if self.graph is None:
             torch.cuda.synchronize(sched.device)
             g = torch.cuda.CUDAGraph()
-            with torch.cuda.graph(g):
+            with graphs.capture(g):
                 self.logits = sched.model.logits(sched.model.forward_tokens(self.tokens, self.batch, sched.caches))
             self.graph = g
         self.graph.replay()

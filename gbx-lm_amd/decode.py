@@ -13,7 +13,7 @@ from typing import List, Optional
 import torch
 import torch.nn.functional as F
 
-from . import env, ops
+from . import env, graphs, ops
 from .models.cache import KVCache
 from .tp import all_reduce_
 
@@ -185,7 +185,7 @@ class DecodeRunner:
         torch.cuda.current_stream(self.dev).wait_stream(s)
         torch.cuda.synchronize(self.dev)
         self.graph = torch.cuda.CUDAGraph()
-        with torch.no_grad(), torch.cuda.graph(self.graph):
+        with torch.no_grad(), graphs.capture(self.graph):
             self.logits = self._forward()
 
     def start_greedy(self, token: torch.Tensor) -> None:
@@ -270,7 +270,7 @@ class GraphDecodeRunner:
         torch.cuda.current_stream(self.dev).wait_stream(side)
         torch.cuda.synchronize(self.dev)
         self.graph = torch.cuda.CUDAGraph()
-        with torch.no_grad(), torch.cuda.graph(self.graph):
+        with torch.no_grad(), graphs.capture(self.graph):
             self.logits = self._forward()
 
     def _forward(self):
@@ -918,7 +918,7 @@ class PromptRunner:
         torch.cuda.current_stream(dev).wait_stream(s)
         torch.cuda.synchronize(dev)
         self.graph = torch.cuda.CUDAGraph()
-        with torch.no_grad(), torch.cuda.graph(self.graph):
+        with torch.no_grad(), graphs.capture(self.graph):
             self.logits = self._forward()
 
     def _forward(self):

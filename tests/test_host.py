@@ -342,3 +342,36 @@ def test_convert_gba_native_repo(tmp_path, double_quant):
         gba2mlx.convert(str(nat), str(out), upload_repo="a/b-mlx")
     big = {f"t{i}": torch.zeros(1 << 20, dtype=torch.float32) for i in range(5)}      # 4 MiB each
     assert [len(s) for s in gba2mlx.make_shards(big, max_file_size_gb=0)] == [0, 1, 1, 1, 1, 1] or len(gba2mlx.make_shards(big)) == 1
+
+
+def test_graph_capture_runs_without_the_garbage_collector(monkeypatch):
+    """No collection may fall into a capture (it could destroy an earlier engine's graph); the collector's state comes back afterwards,
+    also after an error and when it was off before."""
+    import contextlib
+    import gc
+
+    import pytest
+    import torch
+    from gbx_lm_amd import graphs
+    seen = []
+
+    @contextlib.contextmanager
+    def fake(graph, **kwargs):
+        seen.append((graph, gc.isenabled()))
+        yield
+    monkeypatch.setattr(torch.cuda, "graph", fake)
+    assert gc.isenabled()
+    with graphs.capture("g"):
+        assert not gc.isenabled()
+    assert gc.isenabled() and seen == [("g", False)]
+    with pytest.raises(RuntimeError):
+        with graphs.capture("g"):
+            raise RuntimeError("in the capture")
+    assert gc.isenabled()
+    gc.disable()
+    try:
+        with graphs.capture("g"):
+            pass
+        assert not gc.isenabled()
+    finally:
+        gc.enable()
