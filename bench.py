@@ -861,7 +861,7 @@ def main():
     ap.add_argument("--design", default=None, choices=["revitar", "radenex", "tugolix", "laruzen", "leripel"], help="side benchmark of one model design beside the closest existing "
                     "family at equal size (own JSON line; the default workload and its output are unchanged)")
     ap.add_argument("--sizes", default=None, help="--design: comma-separated names of REVITAR_SIZES (default small,a3b-like) / RADENEX_SIZES "
-                    "(default small,lite-like) / TUGOLIX_SIZES (default small,a3b-like)")
+                    "(default small,lite-like) / TUGOLIX_SIZES / LARUZEN_SIZES / LERIPEL_SIZES (default small,a3b-like)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=512, help="timed decode steps (default: > 0.5 s of GPU time, so that a coarse GPU-busy sampler sees the run)")
     ap.add_argument("--warmup", type=int, default=8)
