@@ -329,7 +329,23 @@ class SinkAttnArgs(ctypes.Structure):
                 ("H", ctypes.c_int32), ("G", ctypes.c_int32), ("dk", ctypes.c_int32), ("dv", ctypes.c_int32),
                 ("window", ctypes.c_int32), ("keep", ctypes.c_int32), ("ring", ctypes.c_int32), ("scale", ctypes.c_float),
                 ("decode_only", ctypes.c_int32), ("act", ctypes.c_int32), ("partial", ctypes.c_void_p), ("partial_splits", ctypes.c_int32),
-                ("chunk", ctypes.c_int32), ("head_scale", ctypes.c_void_p), ("out_row", ctypes.c_int64)]
+                ("chunk", ctypes.c_int32), ("head_scale", ctypes.c_void_p), ("out_row", ctypes.c_int64), ("gate_channels", ctypes.c_int32)]
+
+
+class HeadProjectArgs(ctypes.Structure):
+    """Mirror of ``gbxm_head_project_args``."""
+    _fields_ = [("in_", ctypes.c_void_p), ("in_row", ctypes.c_int64), ("in_head", ctypes.c_int64), ("w", ctypes.c_void_p), ("out", ctypes.c_void_p),
+                ("out_row", ctypes.c_int64), ("out_head", ctypes.c_int64), ("gate", ctypes.c_void_p), ("gate_row", ctypes.c_int64),
+                ("positions", ctypes.c_void_p), ("pos_stride", ctypes.c_int64), ("freq", ctypes.c_void_p), ("T", ctypes.c_int64), ("H", ctypes.c_int32),
+                ("n_in", ctypes.c_int32), ("n_out", ctypes.c_int32), ("n_tail", ctypes.c_int32), ("mult", ctypes.c_float),
+                ("interleaved", ctypes.c_int32), ("act", ctypes.c_int32)]
+
+
+class ExpertArgs(ctypes.Structure):
+    """Mirror of ``gbxm_expert_args``."""
+    _fields_ = [("h", ctypes.c_void_p), ("first", ctypes.c_void_p), ("down", ctypes.c_void_p), ("idx", ctypes.c_void_p), ("scale", ctypes.c_void_p),
+                ("y", ctypes.c_void_p), ("T", ctypes.c_int64), ("K", ctypes.c_int32), ("F", ctypes.c_int32), ("E", ctypes.c_int32), ("top", ctypes.c_int32),
+                ("act", ctypes.c_int32), ("kind", ctypes.c_int32), ("limit", ctypes.c_float), ("ws", ctypes.c_void_p), ("ws_bytes", ctypes.c_size_t)]
 
 
 class RecurrentPrepArgs(ctypes.Structure):
@@ -408,7 +424,7 @@ def mixers() -> ctypes.CDLL:
         L.gbxm_window_append.argtypes = [p, i64, i32, i32, i32, p, p, p, p, i64, i32, i32, p]
         L.gbxm_stream_add.argtypes = [p, p, p, i64, i32, p]
         L.gbxm_activate.argtypes = [p, i64, i32, i32, p]
-        L.gbxm_head_project.argtypes = [p, i64, i64, p, p, i64, i64, i64, i32, i32, i32, i32, i32, p]
+        L.gbxm_head_project.argtypes = [ctypes.POINTER(HeadProjectArgs), p]
         L.gbxm_stream_add_norm.argtypes = [p, p, p, p, p, i64, i32, f32, i32, p]
         L.gbxm_rotate_norm_heads.argtypes = [p, i64, i64, p, i64, ctypes.POINTER(HeadSegment), i32, f32, i32, p]
         L.gbxm_slot_append.argtypes = [p, i64, i32, p, i64, i32, p, p, p, p, i64, i32, i32, i32, p]
@@ -418,6 +434,7 @@ def mixers() -> ctypes.CDLL:
         L.gbxm_glu.argtypes = [p, i64, p, i64, p, i64, i64, i32, i32, f32, f32, i32, p]
         L.gbxm_route_sigmoid_groups.argtypes = [p, p, p, p, i64, i32, i32, i32, i32, i32, f32, p]
         L.gbxm_expert_glu_act.argtypes = [p, p, p, p, p, i64, i32, i32, i32, i32, i32, i32, f32, p, sz, p]
+        L.gbxm_expert_ff.argtypes = [ctypes.POINTER(ExpertArgs), p]
         L.gbxm_recurrent_prepare.argtypes = [ctypes.POINTER(RecurrentPrepArgs), p]
         L.gbxm_conv_tail_update.argtypes = [p, i64, p, p, i32, i32, i32, i32, p]
         L.gbxm_state_scan.argtypes = [p, i64, p, p, p, i32, i64, i32, i32, i32, i32, i32, p]
@@ -437,7 +454,7 @@ def mixers() -> ctypes.CDLL:
         L.gbxm_gate_group_norm.argtypes = [p, p, i64, p, p, i64, i64, i32, i32, f32, i32, p]
         L.gbxm_layer_update.argtypes = [ctypes.POINTER(LayerUpdateArgs), p]
         L.gbxm_router_rows.argtypes = [p, p, p, i64, i32, i32, i32, p]
-        L.gbxm_route_groups.argtypes = [p, i64, p, p, i64, i64, i32, i32, i32, i32, i32, p]
+        L.gbxm_route_groups.argtypes = [p, i64, p, p, i64, i64, i32, i32, i32, i32, i32, i32, p]
         _mlib = L
     return _mlib
 

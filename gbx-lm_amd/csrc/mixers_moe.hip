@@ -1,4 +1,6 @@
-// Routed gated MLPs over dense stacked experts:  y[t][s] = down_e (silu(gate_e h_t) * (up_e h_t)),  e = idx[t][s].
+// Routed MLPs over dense stacked experts:  y[t][s] = down_e (silu(gate_e h_t) * (up_e h_t)),  e = idx[t][s] -- or another gated
+// activation, or experts without a gate, down_e relu(up_e h_t)^2.  With a factor per (row, choice) an expert reads the scaled row: the
+// factor meets the fp32 sums of its first products.
 //
 //   * row kernels -- weight-bandwidth bound: the kernels of decode steps, of fp32 models and of shapes the grouped kernel does not
 //     take.  Two launches so that even ONE row spreads over the chip: expert_up_rows (a workgroup = one (row, choice) pair x 8 hidden
@@ -39,9 +41,12 @@ __device__ __forceinline__ float lane_dot(const T* __restrict__ w, const float* 
   return acc;
 }
 
-template <typename T, bool FAST, bool VEC>
-__global__ __launch_bounds__(NT) void expert_up_rows(const T* __restrict__ h, const T* __restrict__ gate_up, const int* __restrict__ idx,
-                                                    T* __restrict__ act, int K, int F, int top, int kind, float limit) {
+// GATED: first = gate rows over up rows, a wave takes one hidden channel at a time; else first = up rows, a wave takes its two channels of
+// the workgroup's FC = 2 NW together.
+template <typename T, bool FAST, bool VEC, bool GATED>
+__global__ __launch_bounds__(NT) void expert_up_rows(const T* __restrict__ h, const T* __restrict__ first, const int* __restrict__ idx,
+                                                    const float* __restrict__ scale, T* __restrict__ act, int K, int F, int top, int kind, float limit) {
+  static_assert(FC == 2 * NW, "two hidden channels per wave");
   extern __shared__ float hl[];                     // the row [K]
   const int64_t pair = blockIdx.x;
   const int e = idx[pair];
@@ -49,12 +54,26 @@ __global__ __launch_bounds__(NT) void expert_up_rows(const T* __restrict__ h, co
   const T* hr = h + (pair / top) * K;
   for (int k = threadIdx.x; k < K; k += NT) hl[k] = to_f32(hr[k]);
   __syncthreads();
-  const T* wg = gate_up + static_cast<int64_t>(e) * 2 * F * K;
+  const T* wg = first + static_cast<int64_t>(e) * (GATED ? 2 : 1) * F * K;
+  const float sc = scale ? scale[pair] : 1.f;
+  if constexpr (!GATED) {
+    const int fa = blockIdx.y * FC + wave, fb = fa + NW;
+    if (fa >= F) return;
+    float a = lane_dot<T, VEC>(wg + static_cast<int64_t>(fa) * K, hl, K, lane);
+    float b = lane_dot<T, VEC>(wg + static_cast<int64_t>(min(fb, F - 1)) * K, hl, K, lane);
+    a = fmaxf(sc * wave_sum(a), 0.f);
+    b = fmaxf(sc * wave_sum(b), 0.f);
+    if (lane == 0) {
+      act[pair * F + fa] = from_f32<T>(a * a);
+      if (fb < F) act[pair * F + fb] = from_f32<T>(b * b);
+    }
+    return;
+  }
   const T* wu = wg + static_cast<int64_t>(F) * K;
   const int f_end = min(F, (static_cast<int>(blockIdx.y) + 1) * FC);
   for (int f = blockIdx.y * FC + wave; f < f_end; f += NW) {
-    const float ag = wave_sum(lane_dot<T, VEC>(wg + static_cast<int64_t>(f) * K, hl, K, lane));
-    const float au = wave_sum(lane_dot<T, VEC>(wu + static_cast<int64_t>(f) * K, hl, K, lane));
+    const float ag = sc * wave_sum(lane_dot<T, VEC>(wg + static_cast<int64_t>(f) * K, hl, K, lane));
+    const float au = sc * wave_sum(lane_dot<T, VEC>(wu + static_cast<int64_t>(f) * K, hl, K, lane));
     if (lane == 0) act[pair * F + f] = from_f32<T>(glu_act<FAST>(ag, au, kind, limit, 1.702f));
   }
 }
@@ -76,31 +95,28 @@ __global__ __launch_bounds__(NT) void expert_down_rows(const T* __restrict__ act
   }
 }
 
+template <typename T, bool FAST, bool VEC, bool GATED>
+int launch_rows(const gbxm_expert_args& a, hipStream_t s) {
+  const int64_t P = a.T * a.top;
+  const dim3 gu(P, (a.F + FC - 1) / FC), gd(P, (a.K + KC - 1) / KC);
+  T* act = static_cast<T*>(a.ws);
+  expert_up_rows<T, FAST, VEC, GATED><<<gu, NT, a.K * sizeof(float), s>>>(static_cast<const T*>(a.h), static_cast<const T*>(a.first), a.idx, a.scale, act, a.K,
+                                                                         a.F, a.top, a.kind, a.limit);
+  expert_down_rows<T, VEC><<<gd, NT, a.F * sizeof(float), s>>>(act, static_cast<const T*>(a.down), a.idx, static_cast<T*>(a.y), a.K, a.F);
+  return after_launch("expert_ff (rows)");
+}
+
 template <typename T, bool FAST>
-int launch_rows(const void* h, const void* gate_up, const void* down, const int32_t* idx, void* y, int64_t P, int K, int F, int top, int kind, float limit,
-                void* ws, hipStream_t s) {
+int launch_rows(const gbxm_expert_args& a, hipStream_t s) {
   constexpr int PER = 16 / sizeof(T);
-  const bool vec = K % PER == 0 && F % PER == 0 &&
-                   (reinterpret_cast<uintptr_t>(gate_up) | reinterpret_cast<uintptr_t>(down)) % 16 == 0;
-  const dim3 gu(P, (F + FC - 1) / FC), gd(P, (K + KC - 1) / KC);
-  const T* hp = static_cast<const T*>(h);
-  const T* gp = static_cast<const T*>(gate_up);
-  const T* dp = static_cast<const T*>(down);
-  T* act = static_cast<T*>(ws);
-  if (vec) {
-    expert_up_rows<T, FAST, true><<<gu, NT, K * sizeof(float), s>>>(hp, gp, idx, act, K, F, top, kind, limit);
-    expert_down_rows<T, true><<<gd, NT, F * sizeof(float), s>>>(act, dp, idx, static_cast<T*>(y), K, F);
-  } else {
-    expert_up_rows<T, FAST, false><<<gu, NT, K * sizeof(float), s>>>(hp, gp, idx, act, K, F, top, kind, limit);
-    expert_down_rows<T, false><<<gd, NT, F * sizeof(float), s>>>(act, dp, idx, static_cast<T*>(y), K, F);
-  }
-  return after_launch("expert_glu (rows)");
+  const bool vec = a.K % PER == 0 && a.F % PER == 0 && (reinterpret_cast<uintptr_t>(a.first) | reinterpret_cast<uintptr_t>(a.down)) % 16 == 0;
+  if (a.kind == GBXM_EXPERT_RELU2) return vec ? launch_rows<T, FAST, true, false>(a, s) : launch_rows<T, FAST, false, false>(a, s);
+  return vec ? launch_rows<T, FAST, true, true>(a, s) : launch_rows<T, FAST, false, true>(a, s);
 }
 
 }  // namespace
 
-int launch_expert_grouped(const void* h, const void* gate_up, const void* down, const int32_t* idx, void* y, int64_t T, int K, int F, int E, int top,
-                          int kind, float limit, void* ws, size_t ws_bytes, hipStream_t s);   // mixers_moe_mfma.hip
+int launch_expert_grouped(const gbxm_expert_args& a, hipStream_t s);   // mixers_moe_mfma.hip
 size_t expert_grouped_workspace(int64_t T, int K, int F, int E, int top);
 
 }  // namespace gbxm
@@ -117,23 +133,29 @@ extern "C" int gbxm_expert_glu_grouped(int64_t T_, int32_t K, int32_t F, int32_t
   return act == GBXM_BF16 && expert_grouped_workspace(T_, K, F, E, top) > 0;
 }
 
+extern "C" int gbxm_expert_ff(const gbxm_expert_args* a, void* stream) {
+  if (!a || !a->h || !a->first || !a->down || !a->idx || !a->y || a->K <= 0 || a->F <= 0 || a->E <= 0 || a->top < 1 || a->top > a->E || a->T < 0 ||
+      (a->act != GBXM_BF16 && a->act != GBXM_F32) || (a->kind != GBXM_GLU_SILU && a->kind != GBXM_GLU_CLAMPED_SWISH && a->kind != GBXM_EXPERT_RELU2))
+    return fail(GBXM_ERR_INVALID, "expert_ff: bad argument");
+  if (a->T == 0) return GBXM_OK;
+  if (!a->ws || a->ws_bytes < gbxm_expert_glu_workspace(a->T, a->K, a->F, a->E, a->top, a->act)) return fail(GBXM_ERR_INVALID, "expert_ff: workspace too small");
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (a->act == GBXM_BF16) {
+    const int rc = launch_expert_grouped(*a, s);
+    if (rc != GBXM_ERR_UNSUPPORTED) return rc;
+  }
+  const int longest = a->K > a->F ? a->K : a->F;
+  if (static_cast<size_t>(longest) * sizeof(float) > 64 * 1024) return fail(GBXM_ERR_UNSUPPORTED, "expert_ff: rows of %d channels beyond the row kernels' LDS", longest);
+  if (a->T * a->top > 0x7fffffffLL || (a->F + FC - 1) / FC > 65535 || (a->K + KC - 1) / KC > 65535) return fail(GBXM_ERR_UNSUPPORTED, "expert_ff: grid");
+  return a->act == GBXM_BF16 ? launch_rows<bf16_t, true>(*a, s) : launch_rows<float, false>(*a, s);
+}
+
 extern "C" int gbxm_expert_glu_act(const void* h, const void* gate_up, const void* down, const int32_t* idx, void* y, int64_t T_, int32_t K,
                                    int32_t F, int32_t E, int32_t top, int32_t act, int32_t kind, float limit, void* ws, size_t ws_bytes,
                                    void* stream) {
-  if (!h || !gate_up || !down || !idx || !y || K <= 0 || F <= 0 || E <= 0 || top < 1 || top > E || T_ < 0 || (act != GBXM_BF16 && act != GBXM_F32) ||
-      (kind != GBXM_GLU_SILU && kind != GBXM_GLU_CLAMPED_SWISH))
-    return fail(GBXM_ERR_INVALID, "expert_glu: bad argument");
-  if (T_ == 0) return GBXM_OK;
-  if (!ws || ws_bytes < gbxm_expert_glu_workspace(T_, K, F, E, top, act)) return fail(GBXM_ERR_INVALID, "expert_glu: workspace too small");
-  hipStream_t s = static_cast<hipStream_t>(stream);
-  if (act == GBXM_BF16) {
-    const int rc = launch_expert_grouped(h, gate_up, down, idx, y, T_, K, F, E, top, kind, limit, ws, ws_bytes, s);
-    if (rc != GBXM_ERR_UNSUPPORTED) return rc;
-  }
-  if (static_cast<size_t>(K > F ? K : F) * sizeof(float) > 64 * 1024) return fail(GBXM_ERR_UNSUPPORTED, "expert_glu: rows of %d channels beyond the row kernels' LDS", K > F ? K : F);
-  if (T_ * top > 0x7fffffffLL || (F + FC - 1) / FC > 65535 || (K + KC - 1) / KC > 65535) return fail(GBXM_ERR_UNSUPPORTED, "expert_glu: grid");
-  return act == GBXM_BF16 ? launch_rows<bf16_t, true>(h, gate_up, down, idx, y, T_ * top, K, F, top, kind, limit, ws, s)
-                          : launch_rows<float, false>(h, gate_up, down, idx, y, T_ * top, K, F, top, kind, limit, ws, s);
+  if (kind == GBXM_EXPERT_RELU2) return fail(GBXM_ERR_INVALID, "expert_glu: gated experts only");
+  const gbxm_expert_args a{h, gate_up, down, idx, nullptr, y, T_, K, F, E, top, act, kind, limit, ws, ws_bytes};
+  return gbxm_expert_ff(&a, stream);
 }
 
 extern "C" int gbxm_expert_glu(const void* h, const void* gate_up, const void* down, const int32_t* idx, void* y, int64_t T_, int32_t K, int32_t F,

@@ -3,7 +3,8 @@
 // 1. expert_sort_kernel: the step's (row, choice) pairs counted and bucketed by expert on the device (one workgroup, LDS counters):
 //    offsets[E + 1], the pair ids in expert order, and the table of row tiles (expert, first pair) the two products walk.  Nothing
 //    returns to the host.
-// 2. expert_up_kernel:   act[p] = silu(gate_e h) * (up_e h) for the pairs of expert e, 128 pairs x 128 hidden channels per workgroup;
+// 2. expert_up_kernel:   act[p] = silu(gate_e h) * (up_e h) for the pairs of expert e, 128 pairs x 128 hidden channels per workgroup (256
+//    where experts have no gate: the second weight fragment is then another block of 32 channels);
 // 3. expert_down_kernel: y[pair] = down_e act[p], 128 pairs x 256 output channels per workgroup.
 // Products are computed swapped -- C^T[channel, pair] = mfma(weight rows, activation rows) -- so a lane ends up with four consecutive
 // channels of one pair (8-byte stores) and the gate / up pair of a channel sits in the same lane for the activation.
@@ -74,19 +75,21 @@ struct BTile {
   }
 };
 
-__global__ __launch_bounds__(256) void expert_up_kernel(const bf16_t* __restrict__ h, const bf16_t* __restrict__ gate_up, const int* __restrict__ offsets,
-                                                       const int* __restrict__ sorted, const int* __restrict__ tile_tab, bf16_t* __restrict__ act,
-                                                       int K, int F, int top, int kind, float limit) {
+template <bool GATED>
+__global__ __launch_bounds__(256) void expert_up_kernel(const bf16_t* __restrict__ h, const bf16_t* __restrict__ first, const int* __restrict__ offsets,
+                                                       const int* __restrict__ sorted, const int* __restrict__ tile_tab, const float* __restrict__ scale,
+                                                       bf16_t* __restrict__ act, int K, int F, int top, int kind, float limit) {
   __shared__ __attribute__((aligned(16))) unsigned char bl[RT * BROW];
   const int bt = xcd_row_tile();
   const int e = tile_tab[2 * bt];
   if (e < 0) return;                                                  // (workgroup-uniform)
   const int lo = tile_tab[2 * bt + 1], hi = offsets[e + 1];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 31, hb = lane >> 5;
-  const int f0 = blockIdx.y * 128 + wave * 32;
+  const int f0 = GATED ? blockIdx.y * 128 + wave * 32 : blockIdx.y * 256 + wave * 64;
   const bool live = f0 < F;                                           // a wave past the last channel still moves its share of the tile
-  const bf16_t* wgl = gate_up + (static_cast<int64_t>(e) * 2 * F + (live ? f0 + r : 0)) * K;
-  const bf16_t* wul = wgl + static_cast<int64_t>(F) * K;
+  const bool second = GATED || f0 + 32 < F;                           // (F is a multiple of 32)
+  const bf16_t* wgl = first + (static_cast<int64_t>(e) * (GATED ? 2 : 1) * F + (live ? f0 + r : 0)) * K;
+  const bf16_t* wul = GATED ? wgl + static_cast<int64_t>(F) * K : (second ? wgl + static_cast<int64_t>(32) * K : wgl);
   BTile b;
   b.cpiece = tid & 7;
 #pragma unroll
@@ -135,13 +138,25 @@ __global__ __launch_bounds__(256) void expert_up_kernel(const bf16_t* __restrict
   for (int j = 0; j < 4; ++j) {
     const int row = lo + j * 32 + r;
     if (row >= hi) continue;
+    const float sc = scale ? scale[sorted[row]] : 1.f;
     bf16_t* ap = act + static_cast<int64_t>(row) * F + f0 + 4 * hb;
 #pragma unroll
     for (int q4 = 0; q4 < 4; ++q4) {
       float v[4];
+      if constexpr (GATED) {
 #pragma unroll
-      for (int i = 0; i < 4; ++i) { const float g = ag[j][4 * q4 + i]; v[i] = glu_act<true>(g, au[j][4 * q4 + i], kind, limit, 1.702f); }
-      *reinterpret_cast<u32x2*>(ap + 8 * q4) = u32x2{pack2(v[0], v[1]), pack2(v[2], v[3])};
+        for (int i = 0; i < 4; ++i) v[i] = glu_act<true>(sc * ag[j][4 * q4 + i], sc * au[j][4 * q4 + i], kind, limit, 1.702f);
+        *reinterpret_cast<u32x2*>(ap + 8 * q4) = u32x2{pack2(v[0], v[1]), pack2(v[2], v[3])};
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) { const float z = fmaxf(sc * ag[j][4 * q4 + i], 0.f); v[i] = z * z; }
+        *reinterpret_cast<u32x2*>(ap + 8 * q4) = u32x2{pack2(v[0], v[1]), pack2(v[2], v[3])};
+        if (second) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) { const float z = fmaxf(sc * au[j][4 * q4 + i], 0.f); v[i] = z * z; }
+          *reinterpret_cast<u32x2*>(ap + 32 + 8 * q4) = u32x2{pack2(v[0], v[1]), pack2(v[2], v[3])};
+        }
+      }
     }
   }
 }
@@ -235,17 +250,17 @@ size_t expert_grouped_workspace(int64_t T, int K, int F, int E, int top) {
   return align16(sizeof(int) * (E + 1)) + align16(sizeof(int) * P) + align16(sizeof(int) * 2 * tiles_of(P, E)) + align16(sizeof(bf16_t) * P * F);
 }
 
-int launch_expert_grouped(const void* h, const void* gate_up, const void* down, const int32_t* idx, void* y, int64_t T, int K, int F, int E, int top,
-                          int kind, float limit, void* ws, size_t ws_bytes, hipStream_t s) {
-  const size_t need = expert_grouped_workspace(T, K, F, E, top);
+int launch_expert_grouped(const gbxm_expert_args& a, hipStream_t s) {
+  const int K = a.K, F = a.F, E = a.E, top = a.top;
+  const size_t need = expert_grouped_workspace(a.T, K, F, E, top);
   if (need == 0) return GBXM_ERR_UNSUPPORTED;
-  if (ws_bytes < need) return fail(GBXM_ERR_INVALID, "expert_glu: workspace of %zu bytes, %zu needed", ws_bytes, need);
-  if ((reinterpret_cast<uintptr_t>(h) | reinterpret_cast<uintptr_t>(gate_up) | reinterpret_cast<uintptr_t>(down) | reinterpret_cast<uintptr_t>(y) |
-       reinterpret_cast<uintptr_t>(ws)) % 16)
+  if (a.ws_bytes < need) return fail(GBXM_ERR_INVALID, "expert_ff: workspace of %zu bytes, %zu needed", a.ws_bytes, need);
+  if ((reinterpret_cast<uintptr_t>(a.h) | reinterpret_cast<uintptr_t>(a.first) | reinterpret_cast<uintptr_t>(a.down) | reinterpret_cast<uintptr_t>(a.y) |
+       reinterpret_cast<uintptr_t>(a.ws)) % 16)
     return GBXM_ERR_UNSUPPORTED;
-  const int P = static_cast<int>(T * top);
+  const int P = static_cast<int>(a.T * top);
   const int tiles = tiles_of(P, E);
-  unsigned char* w = static_cast<unsigned char*>(ws);
+  unsigned char* w = static_cast<unsigned char*>(a.ws);
   int* offsets = reinterpret_cast<int*>(w);
   w += align16(sizeof(int) * (E + 1));
   int* sorted = reinterpret_cast<int*>(w);
@@ -253,12 +268,16 @@ int launch_expert_grouped(const void* h, const void* gate_up, const void* down, 
   int* tile_tab = reinterpret_cast<int*>(w);
   w += align16(sizeof(int) * 2 * tiles);
   bf16_t* act = reinterpret_cast<bf16_t*>(w);
-  expert_sort_kernel<<<1, 1024, (3 * E + 1) * sizeof(int), s>>>(idx, offsets, sorted, tile_tab, tiles, P, E);
-  expert_up_kernel<<<dim3(tiles, (F + 127) / 128), 256, 0, s>>>(static_cast<const bf16_t*>(h), static_cast<const bf16_t*>(gate_up), offsets, sorted,
-                                                                 tile_tab, act, K, F, top, kind, limit);
-  expert_down_kernel<<<dim3(tiles, (K + 255) / 256), 256, 0, s>>>(act, static_cast<const bf16_t*>(down), offsets, sorted, tile_tab,
-                                                                   static_cast<bf16_t*>(y), K, F);
-  return after_launch("expert_glu (grouped)");
+  expert_sort_kernel<<<1, 1024, (3 * E + 1) * sizeof(int), s>>>(a.idx, offsets, sorted, tile_tab, tiles, P, E);
+  const bf16_t* h = static_cast<const bf16_t*>(a.h);
+  const bf16_t* first = static_cast<const bf16_t*>(a.first);
+  if (a.kind == GBXM_EXPERT_RELU2)
+    expert_up_kernel<false><<<dim3(tiles, (F + 255) / 256), 256, 0, s>>>(h, first, offsets, sorted, tile_tab, a.scale, act, K, F, top, a.kind, a.limit);
+  else
+    expert_up_kernel<true><<<dim3(tiles, (F + 127) / 128), 256, 0, s>>>(h, first, offsets, sorted, tile_tab, a.scale, act, K, F, top, a.kind, a.limit);
+  expert_down_kernel<<<dim3(tiles, (K + 255) / 256), 256, 0, s>>>(act, static_cast<const bf16_t*>(a.down), offsets, sorted, tile_tab,
+                                                                   static_cast<bf16_t*>(a.y), K, F);
+  return after_launch("expert_ff (grouped)");
 }
 
 }  // namespace gbxm

@@ -27,7 +27,7 @@ constexpr int DCH = 128;          // value channels per lane pass (two per lane)
 constexpr int NCH = 4;            // lane passes: value sizes up to NCH * DCH
 
 struct SinkGeo {
-  int H, G, dk, dv, window, keep, ring, chunk;
+  int H, G, dk, dv, window, keep, ring, chunk, gate_channels;
   float scale;
   const float* head_scale;
   int64_t out_row;
@@ -207,7 +207,7 @@ __global__ __launch_bounds__(NT) void sink_rows_kernel(const T* __restrict__ q, 
 #pragma unroll
     for (int w = 0; w < NW; ++w) s += sums[w * rc * g.dv + i];
     s /= ll[r];
-    if (gate) s *= sigmoid_<FAST>(to_f32(gate[t * g.gate_row + head0 + r]));
+    if (gate) s *= sigmoid_<FAST>(to_f32(gate[t * g.gate_row + (g.gate_channels ? head0 * g.dv + i : head0 + r)]));
     orow[i] = from_f32<T>(s);
   }
 }
@@ -217,8 +217,8 @@ __global__ __launch_bounds__(NT) void sink_rows_kernel(const T* __restrict__ q, 
 // reads four channels at once; the two halves of the workgroup take the even and the odd splits and meet in LDS.
 template <typename T, bool FAST>
 __global__ __launch_bounds__(256) void sink_reduce_kernel(const float* __restrict__ partial, T* __restrict__ out, const float* __restrict__ sink,
-                                                         const T* __restrict__ gate, int64_t gate_row, int64_t T_, int H, int dv, int splits,
-                                                         int64_t out_row) {
+                                                         const T* __restrict__ gate, int64_t gate_row, int gate_channels, int64_t T_, int H, int dv,
+                                                         int splits, int64_t out_row) {
   __shared__ float wz[64];
   __shared__ float den;
   __shared__ float4 other[128];
@@ -240,7 +240,7 @@ __global__ __launch_bounds__(256) void sink_reduce_kernel(const float* __restric
     if (z == 0) den = l + (sink ? exp_<FAST>(sink[head] - top) : 0.f);
   }
   __syncthreads();
-  const float f = (gate ? sigmoid_<FAST>(to_f32(gate[t * gate_row + head])) : 1.f) / den;
+  const float f = (gate && !gate_channels ? sigmoid_<FAST>(to_f32(gate[t * gate_row + head])) : 1.f) / den;
   const int half = threadIdx.x >> 7, q = threadIdx.x & 127;
   for (int d0 = 0; d0 < dv; d0 += 512) {
     const int d = d0 + 4 * q;
@@ -258,7 +258,9 @@ __global__ __launch_bounds__(256) void sink_reduce_kernel(const float* __restric
     if (!half && d < dv) {
       const float4 u = other[q];
       const float r[4] = {(s.x + u.x) * f, (s.y + u.y) * f, (s.z + u.z) * f, (s.w + u.w) * f};
-      for (int c = 0; c < 4 && d + c < dv; ++c) out[t * out_row + head * dv + d + c] = from_f32<T>(r[c]);
+      for (int c = 0; c < 4 && d + c < dv; ++c)
+        out[t * out_row + head * dv + d + c] =
+            from_f32<T>(gate && gate_channels ? r[c] * sigmoid_<FAST>(to_f32(gate[t * gate_row + head * dv + d + c])) : r[c]);
     }
   }
 }
@@ -291,7 +293,8 @@ int launch_rows(const gbxm_sink_attn_args& a, const SinkGeo& g, int rc, int chun
     sink_rows_kernel<T, FAST, true><<<grid, NT, lds, s>>>(q, kn, vn, kc, vc, a.seq, a.tok, out, a.sink, gate, g, rc, splits, part);
   else
     sink_rows_kernel<T, FAST, false><<<grid, NT, lds, s>>>(q, kn, vn, kc, vc, a.seq, a.tok, out, a.sink, gate, g, rc, splits, part);
-  if (splits > 1) sink_reduce_kernel<T, FAST><<<dim3(a.T, a.H), 256, 0, s>>>(part, out, a.sink, gate, a.gate_row, a.T, a.H, a.dv, splits, g.out_row);
+  if (splits > 1) sink_reduce_kernel<T, FAST><<<dim3(a.T, a.H), 256, 0, s>>>(part, out, a.sink, gate, a.gate_row, a.gate_channels, a.T, a.H, a.dv, splits,
+                                                                                       g.out_row);
   return after_launch("sink_attention (rows)");
 }
 
@@ -300,18 +303,122 @@ struct Segments {
   gbxm_head_segment s[GBXM_MAX_SEGMENTS];
 };
 
-// One workgroup per (row, segment); its waves take the segment's heads four at a time.  A head is staged in LDS as fp32, every
-// lane forms its rotated channels from there (its own and the partner of the pair), the statistic is a wave sum.
+// What a segment needs: nothing but rotations touches the rotated channels only, pair by pair; a plain norm of ONE head (a row part, of any
+// length) is a workgroup's sum; everything else stages heads in LDS.
+enum { SEG_STAGED = 0, SEG_PAIRS = 1, SEG_ROW_NORM = 2 };
+__host__ __device__ __forceinline__ int segment_form(const gbxm_head_segment& g) {
+  if (g.norm == 0) return SEG_PAIRS;
+  return g.heads == 1 && g.rot_dims == 0 ? SEG_ROW_NORM : SEG_STAGED;
+}
+
+// PV neighbouring pairs of a head: (u, w) -> (u cos - w sin, w cos + u sin), channels p[i], p[half + i] or p[2i], p[2i + 1].
+template <typename T, int PV>
+__device__ __forceinline__ void turn_pairs(T* __restrict__ p, int half, bool interleaved, const float* __restrict__ cs, const float* __restrict__ sn) {
+  float u[PV], w[PV];
+  if (interleaved) {
+    float v[2 * PV];
+    if constexpr (PV == 1) {
+      v[0] = to_f32(p[0]); v[1] = to_f32(p[1]);
+    } else {
+      Lanes<T, 4>::load(p, v);
+      Lanes<T, 4>::load(p + 4, v + 4);
+    }
+#pragma unroll
+    for (int i = 0; i < PV; ++i) { u[i] = v[2 * i]; w[i] = v[2 * i + 1]; }
+  } else {
+    Lanes<T, PV>::load(p, u);
+    Lanes<T, PV>::load(p + half, w);
+  }
+  float a[PV], b[PV];
+#pragma unroll
+  for (int i = 0; i < PV; ++i) {
+    a[i] = u[i] * cs[i] - w[i] * sn[i];
+    b[i] = w[i] * cs[i] + u[i] * sn[i];
+  }
+  if (interleaved) {
+    float v[2 * PV];
+#pragma unroll
+    for (int i = 0; i < PV; ++i) { v[2 * i] = a[i]; v[2 * i + 1] = b[i]; }
+    if constexpr (PV == 1) {
+      p[0] = from_f32<T>(v[0]); p[1] = from_f32<T>(v[1]);
+    } else {
+      Lanes<T, 4>::store(p, v);
+      Lanes<T, 4>::store(p + 4, v + 4);
+    }
+  } else {
+    Lanes<T, PV>::store(p, a);
+    Lanes<T, PV>::store(p + half, b);
+  }
+}
+
+// p[0 .. n) -> rms_norm(p) (* w), by the whole workgroup; V channels a thread keeps up to ZN groups of between statistic and result.
+template <typename T, int V>
+__device__ __forceinline__ void row_norm(T* __restrict__ p, int n, const float* __restrict__ w, float eps, float* red) {
+  constexpr int ZN = 4;
+  float z[ZN][V];
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < ZN; ++j) {
+    const int c = (threadIdx.x + j * NT) * V;
+    if (c < n) {
+      Lanes<T, V>::load(p + c, z[j]);
+#pragma unroll
+      for (int i = 0; i < V; ++i) ss += z[j][i] * z[j][i];
+    }
+  }
+  for (int c = (threadIdx.x + ZN * NT) * V; c < n; c += NT * V) {
+    float v[V];
+    Lanes<T, V>::load(p + c, v);
+#pragma unroll
+    for (int i = 0; i < V; ++i) ss += v[i] * v[i];
+  }
+  ss = block_sum<NW>(ss, red);
+  const float r = 1.f / sqrtf(ss / n + eps);
+  auto put = [&](int c, float* v) {
+    if (w) {
+      float g[V];
+      Lanes<float, V>::load(w + c, g);
+#pragma unroll
+      for (int i = 0; i < V; ++i) v[i] *= g[i];
+    }
+#pragma unroll
+    for (int i = 0; i < V; ++i) v[i] *= r;
+    Lanes<T, V>::store(p + c, v);
+  };
+#pragma unroll
+  for (int j = 0; j < ZN; ++j) {
+    const int c = (threadIdx.x + j * NT) * V;
+    if (c < n) put(c, z[j]);
+  }
+  for (int c = (threadIdx.x + ZN * NT) * V; c < n; c += NT * V) {
+    float v[V];
+    Lanes<T, V>::load(p + c, v);
+    put(c, v);
+  }
+}
+
+// One workgroup per (row, segment).  A staged segment: its waves take the heads four at a time.  A head is staged in LDS as fp32, every
+// lane forms its rotated channels from there (its own and the partner of the pair), the statistic is a wave sum.  ``vec``: a bit per
+// segment whose channels and row starts lie on the vector grid.
 template <typename T>
 __global__ __launch_bounds__(NT) void rotate_norm_kernel(T* __restrict__ rows, int64_t stride, const int* __restrict__ positions, int64_t pos_stride,
-                                                        Segments segs, float eps, int max_dim) {
-  extern __shared__ float head_lds[];               // [NW][2][max_dim], then cos [max_dim / 2], sin [max_dim / 2]
+                                                        Segments segs, float eps, int max_dim, int max_half, unsigned vec) {
+  extern __shared__ float head_lds[];               // cos [max_half], sin [max_half], then [NW][2][max_dim]
+  __shared__ float red[NW];
   const gbxm_head_segment sg = segs.s[blockIdx.y];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  float* in = head_lds + wave * 2 * max_dim;
+  const int form = segment_form(sg);
+  if (form == SEG_ROW_NORM) {
+    T* p = rows + blockIdx.x * stride + sg.offset;
+    const float* w = (sg.norm & 1) ? nullptr : sg.weight;
+    if ((vec >> blockIdx.y) & 1) row_norm<T, 4>(p, sg.head_dim, w, eps, red);
+    else row_norm<T, 1>(p, sg.head_dim, w, eps, red);
+    return;
+  }
+  float* cs_t = head_lds;
+  float* sn_t = cs_t + max_half;
+  float* in = sn_t + max_half + wave * 2 * max_dim;
   float* turned = in + max_dim;
-  float* cs_t = head_lds + NW * 2 * max_dim;
-  float* sn_t = cs_t + max_dim / 2 + 1;
   const float pos = static_cast<float>(positions[blockIdx.x * pos_stride]);
   const int half = sg.rot_dims / 2;
   for (int i = threadIdx.x; i < half; i += NT) {    // the row's angles once, for all heads of the segment
@@ -319,6 +426,23 @@ __global__ __launch_bounds__(NT) void rotate_norm_kernel(T* __restrict__ rows, i
     sincosf(pos * sg.freq[i], &sn, &cs);
     cs_t[i] = cs * sg.mult;
     sn_t[i] = sn * sg.mult * sg.sign;
+  }
+  if (form == SEG_PAIRS) {
+    __syncthreads();
+    T* p0 = rows + blockIdx.x * stride + sg.offset + sg.rot_offset;
+    if ((vec >> blockIdx.y) & 1) {
+      const int per = half / 4;
+      for (int i = threadIdx.x; i < sg.heads * per; i += NT) {
+        const int c = (i % per) * 4;
+        turn_pairs<T, 4>(p0 + static_cast<int64_t>(i / per) * sg.head_dim + (sg.interleaved ? 2 * c : c), half, sg.interleaved, cs_t + c, sn_t + c);
+      }
+    } else {
+      for (int i = threadIdx.x; i < sg.heads * half; i += NT) {
+        const int c = i % half;
+        turn_pairs<T, 1>(p0 + static_cast<int64_t>(i / half) * sg.head_dim + (sg.interleaved ? 2 * c : c), half, sg.interleaved, cs_t + c, sn_t + c);
+      }
+    }
+    return;
   }
   for (int h0 = 0; h0 < sg.heads; h0 += NW) {
     const int head = h0 + wave;
@@ -393,16 +517,47 @@ __global__ __launch_bounds__(NT) void stream_add_norm_kernel(float* __restrict__
   for (int c = threadIdx.x; c < width; c += NT) h[t * width + c] = from_f32<T>(xr[c] * r * w[c]);      // (each thread re-reads what it wrote)
 }
 
-// out[t][h][j] = sum_i in[t][h][i] w[h][i][j] for j < n_out, then out[t][h][n_out + c] = in[t][h][n_in + c] for c < n_tail: a small
-// matrix of its own per head, applied to few rows (single-row steps): one workgroup per (row, head), the head's input in LDS,
-// threads across the outputs (coalesced reads of w), fp32 sums.
-template <typename T>
-__global__ __launch_bounds__(NT) void head_project_kernel(const T* __restrict__ in, int64_t in_row, int64_t in_head, const T* __restrict__ w,
-                                                         T* __restrict__ out, int64_t out_row, int64_t out_head, int n_in, int n_out, int n_tail) {
+// out[t][h][j] = sum_i in[t][h][i] w[h][i][j] for j < n_out (times a gate's sigmoid), then out[t][h][n_out + c] = in[t][h][n_in + c] for
+// c < n_tail (copied or turned): a small matrix of its own per head, applied to few rows (single-row steps): one workgroup per (row, head),
+// the head's input in LDS, threads across the outputs (coalesced reads of w), fp32 sums.
+template <typename T, bool FAST>
+struct HeadOut {
+  const gbxm_head_project_args& a;
+  const T* ip;
+  T* op;
+  const T* gp;                                     // this row and head's gates, or null
+  __device__ __forceinline__ HeadOut(const gbxm_head_project_args& a_) : a(a_) {
+    ip = static_cast<const T*>(a.in) + blockIdx.x * a.in_row + blockIdx.y * a.in_head;
+    op = static_cast<T*>(a.out) + blockIdx.x * a.out_row + blockIdx.y * a.out_head;
+    gp = a.gate ? static_cast<const T*>(a.gate) + blockIdx.x * a.gate_row + static_cast<int64_t>(blockIdx.y) * a.n_out : nullptr;
+  }
+  __device__ __forceinline__ void put(int j, float s) const { op[j] = from_f32<T>(gp ? s * sigmoid_<FAST>(to_f32(gp[j])) : s); }
+  __device__ __forceinline__ void tail() const {
+    if (!a.freq) {
+      for (int c = threadIdx.x; c < a.n_tail; c += NT) op[a.n_out + c] = ip[a.n_in + c];
+      return;
+    }
+    const int half = a.n_tail / 2;
+    const float pos = static_cast<float>(a.positions[blockIdx.x * a.pos_stride]);
+    for (int i = threadIdx.x; i < half; i += NT) {
+      const int c0 = a.interleaved ? 2 * i : i, c1 = a.interleaved ? 2 * i + 1 : i + half;
+      float sn, cs;
+      sincosf(pos * a.freq[i], &sn, &cs);
+      sn *= a.mult; cs *= a.mult;
+      const float u = to_f32(ip[a.n_in + c0]), w = to_f32(ip[a.n_in + c1]);
+      op[a.n_out + c0] = from_f32<T>(u * cs - w * sn);
+      op[a.n_out + c1] = from_f32<T>(w * cs + u * sn);
+    }
+  }
+};
+
+template <typename T, bool FAST>
+__global__ __launch_bounds__(NT) void head_project_kernel(const gbxm_head_project_args a) {
   extern __shared__ float xin[];                   // [n_in]
-  const T* ip = in + blockIdx.x * in_row + blockIdx.y * in_head;
-  T* op = out + blockIdx.x * out_row + blockIdx.y * out_head;
-  const T* wp = w + static_cast<int64_t>(blockIdx.y) * n_in * n_out;
+  const HeadOut<T, FAST> o(a);
+  const T* ip = o.ip;
+  const int n_in = a.n_in, n_out = a.n_out;
+  const T* wp = static_cast<const T*>(a.w) + static_cast<int64_t>(blockIdx.y) * n_in * n_out;
   for (int i = threadIdx.x; i < n_in; i += NT) xin[i] = to_f32(ip[i]);
   __syncthreads();
   for (int j = threadIdx.x; j < n_out; j += NT) {
@@ -413,22 +568,22 @@ __global__ __launch_bounds__(NT) void head_project_kernel(const T* __restrict__ 
       for (int u = 0; u < 4; ++u) s4[u] += xin[i + u] * to_f32(wp[static_cast<int64_t>(i + u) * n_out + j]);
     }
     for (; i < n_in; ++i) s4[i & 3] += xin[i] * to_f32(wp[static_cast<int64_t>(i) * n_out + j]);
-    op[j] = from_f32<T>((s4[0] + s4[1]) + (s4[2] + s4[3]));
+    o.put(j, (s4[0] + s4[1]) + (s4[2] + s4[3]));
   }
-  for (int c = threadIdx.x; c < n_tail; c += NT) op[n_out + c] = ip[n_in + c];
+  o.tail();
 }
 
 // The same with 16-byte loads of w: a thread owns a run of PER outputs and every IS-th input channel (IS = 256 / (outputs / PER):
 // all threads stream w, many loads in flight each); the IS partial sums of an output meet in LDS in a fixed order.
-template <typename T>
-__global__ __launch_bounds__(NT) void head_project_vec_kernel(const T* __restrict__ in, int64_t in_row, int64_t in_head, const T* __restrict__ w,
-                                                             T* __restrict__ out, int64_t out_row, int64_t out_head, int n_in, int n_out, int n_tail) {
+template <typename T, bool FAST>
+__global__ __launch_bounds__(NT) void head_project_vec_kernel(const gbxm_head_project_args a) {
   constexpr int PER = 16 / sizeof(T);
   extern __shared__ float xin[];                   // [n_in], then the partial sums [NT * PER]
+  const HeadOut<T, FAST> o(a);
+  const T* ip = o.ip;
+  const int n_in = a.n_in, n_out = a.n_out;
   float* red = xin + n_in;
-  const T* ip = in + blockIdx.x * in_row + blockIdx.y * in_head;
-  T* op = out + blockIdx.x * out_row + blockIdx.y * out_head;
-  const T* wp = w + static_cast<int64_t>(blockIdx.y) * n_in * n_out;
+  const T* wp = static_cast<const T*>(a.w) + static_cast<int64_t>(blockIdx.y) * n_in * n_out;
   const int tid = threadIdx.x;
   for (int i = tid; i < n_in; i += NT) xin[i] = to_f32(ip[i]);
   for (int jb = 0; jb < n_out; jb += NT * PER) {
@@ -464,10 +619,10 @@ __global__ __launch_bounds__(NT) void head_project_vec_kernel(const T* __restric
     for (int j = tid; j < jn; j += NT) {
       float s = 0.f;
       for (int k = 0; k < IS; ++k) s += red[k * jn + j];
-      op[jb + j] = from_f32<T>(s);
+      o.put(jb + j, s);
     }
   }
-  for (int c = tid; c < n_tail; c += NT) op[n_out + c] = ip[n_in + c];
+  o.tail();
 }
 
 __device__ __forceinline__ float activation(float v, int kind) {
@@ -526,7 +681,7 @@ bool sink_tiles_shape(int dk, int dv);
 
 int launch_sink_reduce(const gbxm_sink_attn_args& a, int splits, hipStream_t s) {
   sink_reduce_kernel<bf16_t, true><<<dim3(a.T, a.H), 256, 0, s>>>(static_cast<const float*>(a.partial), static_cast<bf16_t*>(a.out), a.sink,
-                                                                  static_cast<const bf16_t*>(a.gate), a.gate_row, a.T, a.H, a.dv, splits,
+                                                                  static_cast<const bf16_t*>(a.gate), a.gate_row, a.gate_channels, a.T, a.H, a.dv, splits,
                                                                   a.out_row > 0 ? a.out_row : static_cast<int64_t>(a.H) * a.dv);
   return after_launch("sink_attention (join of key splits)");
 }
@@ -560,23 +715,23 @@ int gbxm_stream_add_norm(float* x, const void* a, const void* b, const float* w,
   return after_launch("stream_add_norm");
 }
 
-int gbxm_head_project(const void* in, int64_t in_row, int64_t in_head, const void* w, void* out, int64_t out_row, int64_t out_head, int64_t T_,
-                      int32_t H, int32_t n_in, int32_t n_out, int32_t n_tail, int32_t act, void* stream) {
-  if (!act_ok(act) || !in || !w || !out || T_ < 0 || H < 1 || H > 65535 || n_in < 1 || n_out < 1 || n_tail < 0)
+int gbxm_head_project(const gbxm_head_project_args* a, void* stream) {
+  if (!a || !act_ok(a->act) || !a->in || !a->w || !a->out || a->T < 0 || a->H < 1 || a->H > 65535 || a->n_in < 1 || a->n_out < 1 || a->n_tail < 0 ||
+      (a->freq && (!a->positions || a->n_tail % 2)) || (a->gate && a->gate_row < static_cast<int64_t>(a->H) * a->n_out))
     return fail(GBXM_ERR_INVALID, "head_project: bad argument");
-  if (n_in > 12 * 1024) return fail(GBXM_ERR_UNSUPPORTED, "head_project: %d input channels per head", n_in);
-  if (T_ == 0) return GBXM_OK;
+  if (a->n_in > 12 * 1024) return fail(GBXM_ERR_UNSUPPORTED, "head_project: %d input channels per head", a->n_in);
+  if (a->T == 0) return GBXM_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  const int per = act == GBXM_BF16 ? 8 : 4;
-  if (n_out % per == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0) {
-    GBXM_DISPATCH(act, (head_project_vec_kernel<T><<<dim3(T_, H), NT, (n_in + NT * per) * sizeof(float), s>>>(
-                           static_cast<const T*>(in), in_row, in_head, static_cast<const T*>(w), static_cast<T*>(out), out_row, out_head, n_in, n_out,
-                           n_tail)));
+  const int per = a->act == GBXM_BF16 ? 8 : 4;
+  const dim3 grid(a->T, a->H);
+  if (a->n_out % per == 0 && reinterpret_cast<uintptr_t>(a->w) % 16 == 0) {
+    const size_t lds = (a->n_in + NT * per) * sizeof(float);
+    if (a->act == GBXM_BF16) head_project_vec_kernel<bf16_t, true><<<grid, NT, lds, s>>>(*a);
+    else head_project_vec_kernel<float, false><<<grid, NT, lds, s>>>(*a);
     return after_launch("head_project");
   }
-  GBXM_DISPATCH(act, (head_project_kernel<T><<<dim3(T_, H), NT, n_in * sizeof(float), s>>>(static_cast<const T*>(in), in_row, in_head,
-                                                                                           static_cast<const T*>(w), static_cast<T*>(out), out_row,
-                                                                                           out_head, n_in, n_out, n_tail)));
+  if (a->act == GBXM_BF16) head_project_kernel<bf16_t, true><<<grid, NT, a->n_in * sizeof(float), s>>>(*a);
+  else head_project_kernel<float, false><<<grid, NT, a->n_in * sizeof(float), s>>>(*a);
   return after_launch("head_project");
 }
 
@@ -599,7 +754,8 @@ int gbxm_rotate_norm_heads(void* rows, int64_t T_, int64_t row_stride, const int
   if (!act_ok(act) || !rows || !positions || !segs || n_segs < 1 || n_segs > GBXM_MAX_SEGMENTS || T_ < 0)
     return fail(GBXM_ERR_INVALID, "rotate_norm_heads: bad argument");
   Segments sg{};
-  int max_dim = 0;
+  int max_dim = 0, max_half = 0;
+  unsigned vec = 0;
   for (int i = 0; i < n_segs; ++i) {
     const gbxm_head_segment& g = segs[i];
     if (g.offset < 0 || g.heads < 1 || g.head_dim < 1 || g.offset + static_cast<int64_t>(g.heads) * g.head_dim > row_stride || g.rot_dims < 0 ||
@@ -607,13 +763,21 @@ int gbxm_rotate_norm_heads(void* rows, int64_t T_, int64_t row_stride, const int
         ((g.norm == 2 || g.norm == 4) && !g.weight))
       return fail(GBXM_ERR_INVALID, "rotate_norm_heads: segment %d does not fit its rows", i);
     sg.s[i] = g;
-    max_dim = std::max(max_dim, g.head_dim);
+    const int form = segment_form(g);
+    if (form == SEG_STAGED) max_dim = std::max(max_dim, g.head_dim);
+    max_half = std::max(max_half, g.rot_dims / 2);
+    // groups of four channels (pairs: of four pairs) at 8-byte (bf16) or 16-byte (fp32) addresses
+    const bool base = reinterpret_cast<uintptr_t>(rows) % (act == GBXM_BF16 ? 8 : 16) == 0 && row_stride % 4 == 0 && g.offset % 4 == 0;
+    if (form == SEG_ROW_NORM && base && g.head_dim % 4 == 0 && (!g.weight || reinterpret_cast<uintptr_t>(g.weight) % 16 == 0)) vec |= 1u << i;
+    if (form == SEG_PAIRS && base && g.rot_offset % 4 == 0 && g.head_dim % 4 == 0 && g.rot_dims % 8 == 0) vec |= 1u << i;
   }
-  const size_t lds = (static_cast<size_t>(NW) * 2 * max_dim + 2 * (max_dim / 2 + 1)) * sizeof(float);
+  max_half = (max_half + 3) / 4 * 4;
+  const size_t lds = (static_cast<size_t>(NW) * 2 * max_dim + 2 * max_half) * sizeof(float);
   if (lds > 60 * 1024) return fail(GBXM_ERR_UNSUPPORTED, "rotate_norm_heads: heads of %d channels", max_dim);
   if (T_ == 0) return GBXM_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  GBXM_DISPATCH(act, (rotate_norm_kernel<T><<<dim3(T_, n_segs), NT, lds, s>>>(static_cast<T*>(rows), row_stride, positions, pos_stride, sg, eps, max_dim)));
+  GBXM_DISPATCH(act, (rotate_norm_kernel<T><<<dim3(T_, n_segs), NT, lds, s>>>(static_cast<T*>(rows), row_stride, positions, pos_stride, sg, eps, max_dim, max_half,
+                                                                                  vec)));
   return after_launch("rotate_norm_heads");
 }
 
@@ -653,7 +817,7 @@ int gbxm_sink_attention(const gbxm_sink_attn_args* a, void* stream) {
     const int rc = launch_sink_group(*a, s);
     if (rc != GBXM_ERR_UNSUPPORTED) return rc;
   }
-  SinkGeo g{a->H, a->G, a->dk, a->dv, a->window, a->keep, a->ring, a->chunk, a->scale, a->head_scale,
+  SinkGeo g{a->H, a->G, a->dk, a->dv, a->window, a->keep, a->ring, a->chunk, a->gate_channels, a->scale, a->head_scale,
             a->out_row > 0 ? a->out_row : static_cast<int64_t>(a->H) * a->dv, a->q_row, a->q_head, a->k_row, a->k_head, a->v_row, a->v_head,
             a->kc_slot, a->kc_row, a->kc_head, a->vc_slot, a->vc_row, a->vc_head, a->gate_row};
   const int R = a->H / a->G;

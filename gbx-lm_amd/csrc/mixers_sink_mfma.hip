@@ -35,7 +35,22 @@ struct SinkTileArgs {
   float scale;
   const float* head_scale;
   int64_t out_row;
+  int gate_channels;
 };
+
+// four neighbouring channels of a head's output, times f and (a gate per channel) their gates' sigmoids
+__device__ __forceinline__ u32x2 out4(const SinkTileArgs& a, int64_t row, int head, int d, const f32x16& o, int q4, float f) {
+  float v[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) v[i] = o[4 * q4 + i] * f;
+  if (a.gate_channels) {
+    float g[4];
+    Lanes<bf16_t, 4>::load(a.gate + row * a.gate_row + head * a.dv + d, g);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] *= sigmoid_<true>(g[i]);
+  }
+  return u32x2{pack2(v[0], v[1]), pack2(v[2], v[3])};
+}
 
 template <int DK, int DV>
 __device__ __forceinline__ void sink_tile(const SinkTileArgs& a, const int tile, unsigned char* lds) {
@@ -186,7 +201,7 @@ __device__ __forceinline__ void sink_tile(const SinkTileArgs& a, const int tile,
   if (qvalid) {
     const int64_t row = row0 + tq + qloc;
     float f = 1.f / l;
-    if (a.gate) f *= sigmoid_<true>(to_f32(a.gate[row * a.gate_row + head]));
+    if (a.gate && !a.gate_channels) f *= sigmoid_<true>(to_f32(a.gate[row * a.gate_row + head]));
     bf16_t* op = a.out + row * a.out_row + head * a.dv;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt)
@@ -194,7 +209,7 @@ __device__ __forceinline__ void sink_tile(const SinkTileArgs& a, const int tile,
       for (int q4 = 0; q4 < 4; ++q4) {
         const int d = dt * 32 + 8 * q4 + 4 * hb;
         if (d < a.dv)                                          // dv is a multiple of 8: the four channels are inside together
-          *reinterpret_cast<u32x2*>(op + d) = u32x2{pack2(o[dt][4 * q4] * f, o[dt][4 * q4 + 1] * f), pack2(o[dt][4 * q4 + 2] * f, o[dt][4 * q4 + 3] * f)};
+          *reinterpret_cast<u32x2*>(op + d) = out4(a, row, head, d, o[dt], q4, f);
       }
   }
 }
@@ -377,7 +392,7 @@ __global__ __launch_bounds__(256) void sink_group_kernel(const SinkTileArgs a, c
     return;
   }
   float f = 1.f / l;
-  if (a.gate) f *= sigmoid_<true>(to_f32(a.gate[t * a.gate_row + head]));
+  if (a.gate && !a.gate_channels) f *= sigmoid_<true>(to_f32(a.gate[t * a.gate_row + head]));
   bf16_t* op = a.out + t * a.out_row + head * a.dv;
 #pragma unroll
   for (int i = 0; i < DTW; ++i) {
@@ -387,7 +402,7 @@ __global__ __launch_bounds__(256) void sink_group_kernel(const SinkTileArgs a, c
       for (int q4 = 0; q4 < 4; ++q4) {
         const int d = dt * 32 + 8 * q4 + 4 * hb;
         if (d < a.dv)
-          *reinterpret_cast<u32x2*>(op + d) = u32x2{pack2(o[i][4 * q4] * f, o[i][4 * q4 + 1] * f), pack2(o[i][4 * q4 + 2] * f, o[i][4 * q4 + 3] * f)};
+          *reinterpret_cast<u32x2*>(op + d) = out4(a, t, head, d, o[i], q4, f);
       }
   }
 }
@@ -440,6 +455,7 @@ static bool tile_operands(const gbxm_sink_attn_args& a) {
   if ((a.q_row | a.q_head | a.k_row | a.k_head | a.v_row | a.v_head) % 8 || !aligned16(a.q) || !aligned16(a.k_new) || !aligned16(a.v_new) ||
       !aligned16(a.out) || a.out_row % 8)
     return false;
+  if (a.gate && a.gate_channels && (a.gate_row % 4 || reinterpret_cast<uintptr_t>(a.gate) % 8)) return false;
   if (a.kcache && ((a.kc_slot | a.kc_row | a.kc_head | a.vc_slot | a.vc_row | a.vc_head) % 8 || !aligned16(a.kcache) || !aligned16(a.vcache))) return false;
   return true;
 }
@@ -449,7 +465,7 @@ static SinkTileArgs tile_args(const gbxm_sink_attn_args& a) {
                       static_cast<const bf16_t*>(a.kcache), static_cast<const bf16_t*>(a.vcache), a.seq, a.tiles, static_cast<bf16_t*>(a.out), a.sink,
                       static_cast<const bf16_t*>(a.gate), a.q_row, a.q_head, a.k_row, a.k_head, a.v_row, a.v_head, a.kc_slot, a.kc_row, a.kc_head,
                       a.vc_slot, a.vc_row, a.vc_head, a.gate_row, a.q_tile, a.H, a.G, a.dk, a.dv, a.window, a.keep, a.ring, a.chunk, a.scale, a.head_scale,
-                      a.out_row > 0 ? a.out_row : static_cast<int64_t>(a.H) * a.dv};
+                      a.out_row > 0 ? a.out_row : static_cast<int64_t>(a.H) * a.dv, a.gate && a.gate_channels};
 }
 
 int launch_sink_tiles(const gbxm_sink_attn_args& a, hipStream_t s) {

@@ -4,8 +4,8 @@
 //                         activation dtype, or v's image in the activation dtype at a row stride of the caller's (the input of a
 //                         product over several rows side by side).  One workgroup per row; four neighbouring channels per thread.
 //   router_rows_kernel    fp32 router logits of few rows: a wave per (row, expert), 16-byte loads, sums in a fixed order.
-//   route_groups_kernel   softmax over all experts, the best groups by their largest score, the best experts of those, their scores as
-//                         weights; a column past the experts may hold the logit of a gate whose sigmoid is one more weight.
+//   route_groups_kernel   softmax over all experts (or a sigmoid of each), the best groups by their largest score, the best experts of those,
+//                         their scores as weights; a column past the experts may hold the logit of a gate whose sigmoid is one more weight.
 #include "mixers_common.h"
 
 namespace gbxm {
@@ -20,15 +20,20 @@ __global__ __launch_bounds__(NT) void layer_update_kernel(gbxm_layer_update_args
   __shared__ float ml[64];
   const int64_t t = blockIdx.x;
   const int width = p.width, top = p.top;
-  const T* a = static_cast<const T*>(p.branch) + t * p.branch_row;
+  const T* a = p.branch ? static_cast<const T*>(p.branch) + t * p.branch_row : nullptr;
   const T* cand = p.cand ? static_cast<const T*>(p.cand) + t * top * width : nullptr;
   const T* ex = p.extra ? static_cast<const T*>(p.extra) + t * width : nullptr;
   float* x = p.x + t * width;
-  if (cand && threadIdx.x < top) ml[threadIdx.x] = p.mix[t * p.mix_row + threadIdx.x];
+  if (cand && threadIdx.x < top) ml[threadIdx.x] = p.mix ? p.mix[t * p.mix_row + threadIdx.x] : 1.f;
   __syncthreads();
   auto value = [&](int c, float* v) {
-    Lanes<T, V>::load(a + c, v);
     float u[V];
+    if (a) {
+      Lanes<T, V>::load(a + c, v);
+    } else {
+#pragma unroll
+      for (int i = 0; i < V; ++i) v[i] = 0.f;
+    }
     if (cand)
       for (int k = 0; k < top; ++k) {
         Lanes<T, V>::load(cand + static_cast<int64_t>(k) * width + c, u);
@@ -120,7 +125,7 @@ __global__ __launch_bounds__(NT) void router_rows_kernel(const T* __restrict__ h
 // of it -- larger, or equal with a lower index -- so no round waits for another; ranks are a permutation (a logit that is not a number
 // counts as the smallest).  LDS: candidate logits [E, padded to 4 with -inf], group maxima [n_groups, padded], partial sums.
 __global__ __launch_bounds__(NT) void route_groups_kernel(const float* __restrict__ logits, int64_t row, int* __restrict__ idx, float* __restrict__ weight,
-                                                         int64_t weight_row, int E, int top, int n_groups, int keep_groups, int gate) {
+                                                         int64_t weight_row, int E, int top, int n_groups, int keep_groups, int gate, int sigmoid) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   __shared__ float red[NW];
   float* cl = lds;
@@ -142,6 +147,16 @@ __global__ __launch_bounds__(NT) void route_groups_kernel(const float* __restric
     }
     return rank;
   };
+  if (sigmoid) {                                       // (its order is the logits' order)
+    for (int e = tid; e < E; e += nth) {
+      const int rank = rank_of(cl, (E + 3) / 4, e, cl[e]);
+      if (rank < top) {
+        idx[t * top + rank] = e;
+        weight[t * weight_row + rank] = 1.f / (1.f + expf(-cl[e]));
+      }
+    }
+    return;
+  }
   float mx = -INFINITY;
   for (int e = tid; e < E; e += nth) mx = fmaxf(mx, cl[e]);
 #pragma unroll
@@ -199,14 +214,15 @@ using namespace gbxm;
 extern "C" {
 
 int gbxm_layer_update(const gbxm_layer_update_args* a, void* stream) {
-  if (!a || !act_ok(a->act) || !a->x || !a->branch || a->T < 0 || a->width < 1 || a->branch_row < a->width || (a->cand && (!a->mix || a->top < 1 || a->mix_row < a->top)) ||
+  if (!a || !act_ok(a->act) || !a->x || !(a->branch || a->cand || a->extra) || a->T < 0 || a->width < 1 || (a->branch && a->branch_row < a->width) ||
+      (a->cand && (a->top < 1 || (a->mix && a->mix_row < a->top))) ||
       (a->norm_w && !a->h) || (a->image && a->image_row < a->width))
     return fail(GBXM_ERR_INVALID, "layer_update: bad argument");
   if (a->cand && a->top > 64) return fail(GBXM_ERR_UNSUPPORTED, "layer_update: more than 64 candidate rows");
   if (a->T == 0) return GBXM_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
   const size_t vb = a->act == GBXM_BF16 ? 8 : 16;
-  const bool vec = a->width % 4 == 0 && a->branch_row % 4 == 0 && aligned(a->x, 16) && aligned(a->branch, vb) && (!a->cand || aligned(a->cand, vb)) &&
+  const bool vec = a->width % 4 == 0 && aligned(a->x, 16) && (!a->branch || (a->branch_row % 4 == 0 && aligned(a->branch, vb))) && (!a->cand || aligned(a->cand, vb)) &&
                    (!a->extra || aligned(a->extra, vb)) && (!a->norm_w || (aligned(a->norm_w, 16) && aligned(a->h, vb))) &&
                    (!a->image || (a->image_row % 4 == 0 && aligned(a->image, vb)));
   if (a->act == GBXM_BF16) {
@@ -237,15 +253,16 @@ int gbxm_router_rows(const void* h, const float* router, float* logits, int64_t 
 }
 
 int gbxm_route_groups(const float* logits, int64_t row, int32_t* idx, float* weight, int64_t weight_row, int64_t T_, int32_t E, int32_t top, int32_t n_groups,
-                      int32_t keep_groups, int32_t gate, void* stream) {
-  if (!logits || !idx || !weight || E < 1 || top < 1 || top > E || T_ < 0 || row < E + (gate ? 1 : 0) || weight_row < top + (gate ? 1 : 0) || n_groups < 0 ||
+                      int32_t keep_groups, int32_t gate, int32_t sigmoid, void* stream) {
+  if (!logits || (sigmoid && (n_groups || gate)) || !idx || !weight || E < 1 || top < 1 || top > E || T_ < 0 || row < E + (gate ? 1 : 0) || weight_row < top + (gate ? 1 : 0) || n_groups < 0 ||
       (n_groups > 0 && (E % n_groups || keep_groups < 1 || keep_groups > n_groups || top > keep_groups * (E / n_groups))))
     return fail(GBXM_ERR_INVALID, "route_groups: bad argument");
   if (E > 8192) return fail(GBXM_ERR_UNSUPPORTED, "route_groups: more than 8192 experts");
   if (T_ == 0) return GBXM_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
   const size_t lds = ((E + 3) / 4 * 4 + (n_groups + 3) / 4 * 4 + 4) * sizeof(float);
-  route_groups_kernel<<<dim3(T_), E <= 64 ? 64 : (E <= 128 ? 128 : NT), lds, s>>>(logits, row, idx, weight, weight_row, E, top, n_groups, keep_groups, gate);
+  route_groups_kernel<<<dim3(T_), E <= 64 ? 64 : (E <= 128 ? 128 : NT), lds, s>>>(logits, row, idx, weight, weight_row, E, top, n_groups, keep_groups, gate,
+                                                                                          sigmoid);
   return after_launch("route_groups");
 }
 

@@ -104,23 +104,31 @@ def route_topk(h: torch.Tensor, router: torch.Tensor, top: int, renormalize: boo
 _GLU = {"silu": 1, "clamped_swish": 2, "gelu_tanh": 3, "sigmoid": 4}
 
 
+_EXPERT = {"silu": 1, "clamped_swish": 2, "relu2": 16}
+
+
 def expert_glu(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, idx: torch.Tensor, activation: str = "silu",
-               limit: float = 0.0) -> torch.Tensor:
+               limit: float = 0.0, scale: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """The chosen experts' outputs [T, top, K]; ``activation`` "relu2": experts without a gate (``gate_up`` [E, F, K] is up alone);
+    ``scale`` fp32 [T, top]: an expert reads its row times this factor."""
     act = _act(h, "h")
     h = h.contiguous()
     t, k = h.shape
     e, f2, k2 = gate_up.shape
-    f, top = f2 // 2, idx.shape[1]
+    f, top = (f2 if activation == "relu2" else f2 // 2), idx.shape[1]
     if k2 != k or tuple(down.shape) != (e, k, f) or gate_up.dtype != h.dtype or down.dtype != h.dtype or idx.dtype != torch.int32:
         raise ValueError("expert_glu: weights do not fit the rows")
     if not (gate_up.is_contiguous() and down.is_contiguous() and idx.is_contiguous()):
         raise ValueError("expert_glu: contiguous operands")
+    if scale is not None and scale.shape != (t, top):
+        raise ValueError("expert_glu: one input factor per row and choice")
     y = torch.empty((t, top, k), dtype=h.dtype, device=h.device)
     L = _lib.mixers()
     nbytes = L.gbxm_expert_glu_workspace(t, k, f, e, top, act)
     ws = torch.empty((nbytes,), dtype=torch.uint8, device=h.device) if nbytes else None
-    _lib.check_mixers(L.gbxm_expert_glu_act(h.data_ptr(), gate_up.data_ptr(), down.data_ptr(), idx.data_ptr(), y.data_ptr(), t, k, f, e, top, act,
-                                            _GLU[activation], float(limit), None if ws is None else ws.data_ptr(), nbytes, _stream(h.device)))
+    a = _lib.ExpertArgs(h.data_ptr(), gate_up.data_ptr(), down.data_ptr(), idx.data_ptr(), None if scale is None else _f32(scale, "scale").data_ptr(),
+                        y.data_ptr(), t, k, f, e, top, act, _EXPERT[activation], float(limit), None if ws is None else ws.data_ptr(), nbytes)
+    _lib.check_mixers(L.gbxm_expert_ff(ctypes.byref(a), _stream(h.device)))
     return y
 
 
@@ -183,17 +191,33 @@ def stream_add_norm_(x: torch.Tensor, a: torch.Tensor, b: Optional[torch.Tensor]
     return h
 
 
-def head_project(x: torch.Tensor, w: torch.Tensor, n_tail: int = 0) -> torch.Tensor:
+def head_project(x: torch.Tensor, w: torch.Tensor, n_tail: int = 0, turn=None, positions: Optional[torch.Tensor] = None,
+                 gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """x [T, H, n_in + n_tail] (unit channel stride), w [H, n_in, n_out] -> [T, H, n_out + n_tail]: every head's own matrix on its
-    first n_in channels, the tail copied through.  For the few rows of decode steps (one workgroup per row and head)."""
+    first n_in channels (times sigmoid(gate [T, H * n_out])), the tail copied through or turned as ``turn`` (a ``HeadSegment`` of x's
+    heads) says.  For the few rows of decode steps (one workgroup per row and head)."""
     act = _act(x, "x")
     t, heads, width = x.shape
     n_in, n_out = w.shape[1], w.shape[2]
     if w.shape[0] != heads or width != n_in + n_tail or x.stride(2) != 1 or w.dtype != x.dtype or not w.is_contiguous():
         raise ValueError("head_project: operands do not fit")
     out = torch.empty((t, heads, n_out + n_tail), dtype=x.dtype, device=x.device)
-    _lib.check_mixers(_lib.mixers().gbxm_head_project(x.data_ptr(), x.stride(0), x.stride(1), w.data_ptr(), out.data_ptr(), out.stride(0), out.stride(1),
-                                                     t, heads, n_in, n_out, n_tail, act, _stream(x.device)))
+    a = _lib.HeadProjectArgs()
+    a.in_, a.in_row, a.in_head, a.w = x.data_ptr(), x.stride(0), x.stride(1), w.data_ptr()
+    a.out, a.out_row, a.out_head = out.data_ptr(), out.stride(0), out.stride(1)
+    if gate is not None:
+        if n_tail or gate.shape != (t, heads * n_out) or gate.stride(1) != 1 or gate.dtype != x.dtype:
+            raise ValueError("head_project: a gate per output channel, in the rows' dtype, and no tail")
+        a.gate, a.gate_row = gate.data_ptr(), max(gate.stride(0), heads * n_out)
+    if turn is not None:
+        if (turn.rot_offset, turn.rot_dims, turn.norm, turn.sign) != (n_in, n_tail, 0, 1.0) or turn.freq.numel() != n_tail // 2:
+            raise ValueError("head_project: the tail is what turns, and nothing else happens to it")
+        if positions is None or positions.dtype != torch.int32 or positions.shape != (t,):
+            raise ValueError("head_project: int32 positions [T]")
+        a.positions, a.pos_stride, a.freq = positions.data_ptr(), positions.stride(0), _f32(turn.freq, "freq").data_ptr()
+        a.mult, a.interleaved = float(turn.mult), int(turn.interleaved)
+    a.T, a.H, a.n_in, a.n_out, a.n_tail, a.act = t, heads, n_in, n_out, n_tail, act
+    _lib.check_mixers(_lib.mixers().gbxm_head_project(ctypes.byref(a), _stream(x.device)))
     return out
 
 
@@ -255,8 +279,8 @@ def sink_attention(q: torch.Tensor, k_new: torch.Tensor, v_new: torch.Tensor, ca
         raise ValueError("sink_attention: q / k / v do not fit the step")
     if sink is not None and sink.numel() != heads:
         raise ValueError("sink_attention: one sink per head")
-    if gate is not None and (gate.shape != (t, heads) or gate.stride(1) != 1 or gate.dtype != q.dtype):
-        raise ValueError("sink_attention: gate [T, H] in the activation dtype")
+    if gate is not None and (gate.shape not in ((t, heads), (t, heads * dv)) or gate.stride(1) != 1 or gate.dtype != q.dtype):
+        raise ValueError("sink_attention: gate [T, H] or [T, H * dv] in the activation dtype")
     a = _lib.SinkAttnArgs()
     a.q, a.q_row, a.q_head = q.data_ptr(), q.stride(0), q.stride(1)
     a.k_new, a.k_row, a.k_head = k_new.data_ptr(), k_new.stride(0), k_new.stride(1)
@@ -264,12 +288,14 @@ def sink_attention(q: torch.Tensor, k_new: torch.Tensor, v_new: torch.Tensor, ca
     longest = max(p + n for p, n in zip(batch.pos0, batch.n_new))
     if cache is not None and cache.keys is not None:
         kc, vc = cache.keys, cache.values
-        if kc.dtype != q.dtype or kc.shape[0] <= max(batch.slot) or kc.shape[2] < groups * dk or vc.shape[2] < groups * dv:
+        k_head, v_head = (dk, dv) if cache.head_row is None else (cache.head_row, cache.head_row)
+        if (kc.dtype != q.dtype or kc.shape[0] <= max(batch.slot) or kc.shape[2] < (groups - 1) * k_head + cache.key_off + dk
+                or vc.shape[2] < (groups - 1) * v_head + dv):
             raise ValueError("sink_attention: the table does not fit the step")
         if cache.window is None and chunk is None and cache.ring < longest:
             raise ValueError("sink_attention: the table is shorter than the step's longest sequence")
-        a.kcache, a.kc_slot, a.kc_row, a.kc_head = kc.data_ptr(), kc.stride(0), kc.stride(1), dk
-        a.vcache, a.vc_slot, a.vc_row, a.vc_head = vc.data_ptr(), vc.stride(0), vc.stride(1), dv
+        a.kcache, a.kc_slot, a.kc_row, a.kc_head = kc.data_ptr() + cache.key_off * kc.element_size(), kc.stride(0), kc.stride(1), k_head
+        a.vcache, a.vc_slot, a.vc_row, a.vc_head = vc.data_ptr(), vc.stride(0), vc.stride(1), v_head
         a.keep, a.ring = cache.keep, cache.ring
     else:
         if any(batch.pos0):
@@ -289,7 +315,7 @@ def sink_attention(q: torch.Tensor, k_new: torch.Tensor, v_new: torch.Tensor, ca
     a.out = out.data_ptr()
     a.sink = _f32(sink, "sink").data_ptr() if sink is not None else None
     if gate is not None:
-        a.gate, a.gate_row = gate.data_ptr(), gate.stride(0)
+        a.gate, a.gate_row, a.gate_channels = gate.data_ptr(), gate.stride(0), int(gate.shape[1] != heads)
     a.T, a.B, a.n_tiles, a.q_tile = t, len(batch.slot), 0 if batch.tiles is None else batch.tiles.shape[0], batch.q_tile
     a.H, a.G, a.dk, a.dv = heads, groups, dk, dv
     a.window, a.scale = (0 if window is None else int(window)), float(scale)
@@ -654,30 +680,42 @@ def gate_group_norm(o: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, grou
 
 
 # ------------------------------------------------------------------------------- parallel layers with routed experts
-def layer_update_(x: torch.Tensor, branch: torch.Tensor, cand: Optional[torch.Tensor], mix: Optional[torch.Tensor], norm_w: Optional[torch.Tensor],
-                  eps: float, image: Optional[torch.Tensor], replace: bool) -> Optional[torch.Tensor]:
-    """models/residual.py:layer_update_ as one launch; ``mix`` fp32 [T, >= top]: the first ``top`` columns weigh the candidates."""
-    act = _act(branch, "branch")
+def layer_update_(x: torch.Tensor, branch: Optional[torch.Tensor], cand: Optional[torch.Tensor], mix: Optional[torch.Tensor], norm_w: Optional[torch.Tensor],
+                  eps: float, image: Optional[torch.Tensor], replace: bool, extra: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """models/residual.py:layer_update_ as one launch; ``mix`` fp32 [T, >= top]: the first ``top`` columns weigh the candidates (None: 1)."""
+    parts = [p for p in (branch, cand, extra) if p is not None]
+    if not parts or any(p.dtype != parts[0].dtype for p in parts):
+        raise ValueError("layer_update_: at least one part, all of the activation dtype")
+    dtype = parts[0].dtype
+    act = _act(parts[0], "branch")
     _f32(x, "x")
     t, width = x.shape
-    if branch.shape != (t, width) or branch.stride(1) != 1:
-        raise ValueError("layer_update_: the branch is [T, W]")
     a = _lib.LayerUpdateArgs()
-    a.x, a.branch, a.branch_row, a.top = x.data_ptr(), branch.data_ptr(), max(branch.stride(0), width), 0
+    a.x, a.top = x.data_ptr(), 0
+    if branch is not None:
+        if branch.shape != (t, width) or branch.stride(1) != 1:
+            raise ValueError("layer_update_: the branch is [T, W]")
+        a.branch, a.branch_row = branch.data_ptr(), max(branch.stride(0), width)
     if cand is not None:
-        if cand.dtype != branch.dtype or cand.dim() != 3 or cand.shape[0] != t or cand.shape[2] != width or not cand.is_contiguous():
+        if cand.dim() != 3 or cand.shape[0] != t or cand.shape[2] != width or not cand.is_contiguous():
             raise ValueError("layer_update_: candidates [T, top, W] in the activation dtype")
-        if mix.dtype != torch.float32 or mix.shape[0] != t or mix.shape[1] < cand.shape[1] or mix.stride(1) != 1:
-            raise ValueError("layer_update_: a weight per candidate")
-        a.cand, a.top, a.mix, a.mix_row = cand.data_ptr(), cand.shape[1], mix.data_ptr(), max(mix.stride(0), mix.shape[1])
+        a.cand, a.top = cand.data_ptr(), cand.shape[1]
+        if mix is not None:
+            if mix.dtype != torch.float32 or mix.shape[0] != t or mix.shape[1] < cand.shape[1] or mix.stride(1) != 1:
+                raise ValueError("layer_update_: a weight per candidate")
+            a.mix, a.mix_row = mix.data_ptr(), max(mix.stride(0), mix.shape[1])
+    if extra is not None:
+        if extra.shape != (t, width) or not extra.is_contiguous():
+            raise ValueError("layer_update_: the extra rows are contiguous [T, W]")
+        a.extra = extra.data_ptr()
     h = None
     if norm_w is not None:
         if norm_w.numel() != width:
             raise ValueError("layer_update_: one norm weight per channel")
-        h = torch.empty((t, width), dtype=branch.dtype, device=x.device)
+        h = torch.empty((t, width), dtype=dtype, device=x.device)
         a.norm_w, a.h = _f32(norm_w, "norm_w").data_ptr(), h.data_ptr()
     if image is not None:
-        if image.shape != (t, width) or image.dtype != branch.dtype or image.stride(1) != 1:
+        if image.shape != (t, width) or image.dtype != dtype or image.stride(1) != 1:
             raise ValueError("layer_update_: image rows do not fit")
         a.image, a.image_row = image.data_ptr(), max(image.stride(0), width)
     a.T, a.width, a.replace, a.eps, a.act = t, width, int(bool(replace)), float(eps), act
@@ -685,9 +723,10 @@ def layer_update_(x: torch.Tensor, branch: torch.Tensor, cand: Optional[torch.Te
     return h
 
 
-def route_groups(h: torch.Tensor, router: torch.Tensor, experts: int, top: int, groups):
+def route_groups(h: torch.Tensor, router: torch.Tensor, experts: int, top: int, groups, sigmoid: bool = False):
     """(idx int32 [T, top], weights fp32 [T, top (+ 1)]).  ``router`` fp32 [experts (+ 1), W]: a row past the experts is a gate's, whose sigmoid
-    is the last weight.  Logits in fp32: few rows one HIP launch, prompt-sized steps the vendor library's product."""
+    is the last weight.  ``sigmoid`` (no groups, no gate row): scores are sigmoids of the logits instead of their softmax.  Logits in fp32:
+    few rows one HIP launch, prompt-sized steps the vendor library's product."""
     act = _act(h, "h")
     t, rows = h.shape[0], router.shape[0]
     gate = rows - experts
@@ -704,5 +743,5 @@ def route_groups(h: torch.Tensor, router: torch.Tensor, experts: int, top: int, 
     w = torch.empty((t, top + gate), dtype=torch.float32, device=h.device)
     count, keep = groups if groups is not None else (0, 0)
     _lib.check_mixers(_lib.mixers().gbxm_route_groups(logits.data_ptr(), rows, idx.data_ptr(), w.data_ptr(), top + gate, t, experts, top, count, keep, gate,
-                                                     _stream(h.device)))
+                                                     int(bool(sigmoid)), _stream(h.device)))
     return idx, w

@@ -177,12 +177,17 @@ class SlotKVCache:
     * no window (``window=None``): ``keep = 0`` and the ring is the whole capacity, which doubles when a sequence outgrows it
       (row = position while it fits, so a larger table is the old one copied in front).
 
-    ``v_width = 0`` stores one row per token only (a mixer whose values are a part of its key rows: ``values`` is ``keys``).  As
-    with ``WindowKVCache`` a step's own tokens are read from the step and appended after it has attended."""
+    ``v_width = 0`` stores one row per token only (a mixer whose values are a part of its key rows: ``values`` is ``keys``).
+    ``head_row``: channels from one key/value head to the next inside a row (None: the heads of keys and of values lie packed); a
+    head's key starts ``key_off`` channels behind its start, its value at the start.  As with ``WindowKVCache`` a step's own tokens
+    are read from the step and appended after it has attended."""
 
     def __init__(self, k_width: int, v_width: int, window: Optional[int], keep: int = 0, slots: Optional[SequenceSlots] = None,
-                 first_capacity: int = 256):
+                 first_capacity: int = 256, head_row: Optional[int] = None, key_off: int = 0):
         self.k_width, self.v_width = int(k_width), int(v_width)
+        self.head_row, self.key_off = (None if head_row is None else int(head_row)), int(key_off)
+        if self.key_off and self.head_row is None:
+            raise ValueError("SlotKVCache: a key offset goes with head_row")
         self.window = None if window is None else int(window)
         self.keep = 0 if window is None else min(int(keep), 1 << 30)
         self.ring = first_capacity if window is None else self.window
@@ -233,6 +238,13 @@ class SlotKVCache:
             self.keys[:old_k.shape[0]] = old_k
             if self.v_width:
                 self.values[:old_v.shape[0]] = old_v
+
+    def heads_of(self, slot: int, rows: torch.Tensor, groups: int, dk: int, dv: int):
+        """(keys [n, groups, dk], values [n, groups, dv]) of a slot's rows."""
+        def pick(table, at, n):
+            step = n if self.head_row is None else self.head_row
+            return table[slot, rows].as_strided((rows.numel(), groups, n), (table.shape[2], step, 1), at)
+        return pick(self.keys, self.key_off, dk), pick(self.values, 0, dv)
 
     def stored(self, pos0: int) -> torch.Tensor:
         """Positions before ``pos0`` whose rows are still in the table, ascending."""

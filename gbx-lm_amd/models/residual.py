@@ -163,21 +163,25 @@ def normed_pair_mean(a: torch.Tensor, b: torch.Tensor, wa: torch.Tensor, wb: tor
     return (0.5 * (na + nb)).to(a.dtype)
 
 
-def layer_update_(x: torch.Tensor, branch: torch.Tensor, cand: Optional[torch.Tensor], mix: Optional[torch.Tensor], norm: Optional["StreamRMSNorm"],
-                  image: Optional[torch.Tensor] = None, replace: bool = False) -> Optional[torch.Tensor]:
+def layer_update_(x: torch.Tensor, branch: Optional[torch.Tensor], cand: Optional[torch.Tensor], mix: Optional[torch.Tensor], norm: Optional["StreamRMSNorm"],
+                  image: Optional[torch.Tensor] = None, replace: bool = False, extra: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """v = (x, or 0 with ``replace``) + branch [T, W] + sum_k mix[t, k] cand[t, k] (candidates [T, top, W] with fp32 weights, of which the first
-    ``top`` columns are used; None: no candidates), in fp32; the stream ``x`` becomes v in place.  Then ``norm`` of v in the branch's dtype
-    is returned, and / or v's image in that dtype is written to ``image`` [T, W] (any row stride).  GPU tensors: one launch."""
+    ``top`` columns are used, or each with weight 1 when ``mix`` is None) + extra [T, W], in fp32, each part optional but one; the stream
+    ``x`` becomes v in place.  Then ``norm`` of v in the parts' dtype is returned, and / or v's image in that dtype is written to
+    ``image`` [T, W] (any row stride).  GPU tensors: one launch."""
     if x.is_cuda:
         from .. import mixer_ops as M
-        return M.layer_update_(x, branch, cand, mix, None if norm is None else norm.weight, 0.0 if norm is None else norm.eps, image, replace)
-    v = branch.float()
+        return M.layer_update_(x, branch, cand, mix, None if norm is None else norm.weight, 0.0 if norm is None else norm.eps, image, replace, extra)
+    act = next(p for p in (branch, cand, extra) if p is not None).dtype
+    v = torch.zeros_like(x) if branch is None else branch.float()
     if cand is not None:
-        v = v + (cand.float() * mix.float()[:, :cand.shape[1], None]).sum(1)
+        v = v + (cand.float() if mix is None else cand.float() * mix.float()[:, :cand.shape[1], None]).sum(1)
+    if extra is not None:
+        v = v + extra.float()
     if replace:
         x.copy_(v)
     else:
         x.add_(v)
     if image is not None:
         image.copy_(x.to(image.dtype))
-    return None if norm is None else norm(x, branch.dtype)
+    return None if norm is None else norm(x, act)

@@ -18,11 +18,14 @@ Mixers:
   channels, any frequency table) and then set to unit root mean square per head; values are rotated by their own position over all
   of their channels and cached so, a head's output is turned back by the query's position (so a value enters rotated by the
   distance); window with kept first tokens; sink 0.
+* ``SharedKeyValueAttention``: grouped-query attention over all earlier keys whose values are the key projections before they are
+  rotated; sink 0.  A table row holds every channel of a key head once, and the rotated ones a second time.
 * ``LatentAttention``: keys and values of all heads are products of one small latent row per token, ``c = norm(W_dkv h)``, plus one
   rotated key part shared by all heads; only ``c | rotated part`` is cached.  Whole prompts form every head's keys and values from
   ``c`` and attend as usual; steps with history attend over the cached rows directly: the key product is moved to the query side
   (``q' = W_uk^T q``), the value product behind the weighted sum (``o = W_uv sum_j p_j c_j``) -- one shared key/value row of
-  ``kv_rank + rot_dim`` channels for all heads.  Learned sink per head, sigmoid output gate from the mixer's input.
+  ``kv_rank + rot_dim`` channels for all heads.  Learned sink per head, sigmoid output gate from the mixer's input (per head or per
+  channel); queries as one product or through a normed latent of their own.
 
 GPU tensors run the HIP kernels of ``mixer_ops``; CPU tensors the plain torch graph below, which the kernels are tested against.
 """
@@ -120,14 +123,15 @@ def _attend_one(q, k, v, pos_q, pos_k, scale, window, keep, sink, gate, chunk=No
         den = den + torch.exp(sink.float()[:, None, None] - top)
     o = torch.matmul(e / den, vh).transpose(0, 1)                                         # [n, H, dv]
     if gate is not None:
-        o = o * torch.sigmoid(gate.float())[:, :, None]
+        g = torch.sigmoid(gate.float())
+        o = o * (g[:, :, None] if g.shape[1] == heads else g.view(o.shape))
     return o
 
 
 def sink_attend(q: torch.Tensor, k_new: torch.Tensor, v_new: torch.Tensor, cache: Optional[SlotKVCache], batch, scale: float,
                 window: Optional[int], keep: int, sink: Optional[torch.Tensor], gate: Optional[torch.Tensor] = None, chunk: Optional[int] = None,
                 head_scale: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """q [T, H, dk], k_new [T, G, dk], v_new [T, G, dv] (views with unit inner stride), gate [T, H] or None -> [T, H * dv].
+    """q [T, H, dk], k_new [T, G, dk], v_new [T, G, dv] (views with unit inner stride), gate [T, H], [T, H * dv] or None -> [T, H * dv].
     ``cache`` (or None when no sequence of the step has history) holds the positions before the step; with ``chunk`` its table is one
     of ``window = chunk`` rows.  ``head_scale`` fp32 [H]; ``out``: rows to write into (any row stride)."""
     if q.is_cuda:
@@ -144,8 +148,8 @@ def sink_attend(q: torch.Tensor, k_new: torch.Tensor, v_new: torch.Tensor, cache
         if pos0:
             old = cache.stored(pos0)
             rows = cache.row_of(old)
-            k = torch.cat([cache.keys[slot, rows, :groups * k.shape[2]].float().view(-1, groups, k.shape[2]), k])
-            v = torch.cat([cache.values[slot, rows, :groups * dv].float().view(-1, groups, dv), v])
+            k_old, v_old = cache.heads_of(slot, rows, groups, k.shape[2], dv)
+            k, v = torch.cat([k_old.float(), k]), torch.cat([v_old.float(), v])
             pos_k = torch.cat([old, pos_k])
         o = _attend_one(q[r0:r0 + n].float(), k, v, torch.arange(pos0, pos0 + n), pos_k, scale, window, keep, sink,
                         None if gate is None else gate[r0:r0 + n], chunk, head_scale)
@@ -154,14 +158,22 @@ def sink_attend(q: torch.Tensor, k_new: torch.Tensor, v_new: torch.Tensor, cache
     return out
 
 
-def head_project(x: torch.Tensor, w: torch.Tensor, n_tail: int = 0) -> torch.Tensor:
+def head_project(x: torch.Tensor, w: torch.Tensor, n_tail: int = 0, turn: Optional[HeadSegment] = None, positions: Optional[torch.Tensor] = None,
+                 gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """x [T, H, n_in + n_tail], w [H, n_in, n_out] -> [T, H, n_out + n_tail]: each head's own matrix on its first n_in channels, the
-    remaining channels copied through.  Few GPU rows: one HIP launch; else a batched matrix product."""
+    remaining channels copied through -- or, with ``turn`` (a segment that describes x's heads with rot_offset = n_in, rot_dims =
+    n_tail) and ``positions`` int32 [T], rotated.  ``gate`` [T, H * n_out] (no tail): every channel times its sigmoid.  Few GPU rows: one
+    HIP launch; else a batched matrix product (and the row launches for rotation and gate, in place on x and on the product)."""
     if x.is_cuda and x.shape[0] <= 32:
         from .. import mixer_ops as M
-        return M.head_project(x, w, n_tail)
+        return M.head_project(x, w, n_tail, turn, positions, gate)
     n_in = w.shape[1]
+    if turn is not None:
+        rotate_norm_heads_(x.flatten(1), positions, [turn], 0.0)
     y = torch.bmm(x[:, :, :n_in].transpose(0, 1), w).transpose(0, 1)
+    if gate is not None:
+        from .feed_forward import gate_mul
+        return gate_mul(gate, y.reshape(y.shape[0], -1), "sigmoid").view(y.shape)
     return torch.cat([y, x[:, :, n_in:]], dim=-1) if n_tail else y.contiguous()
 
 
@@ -324,25 +336,88 @@ class ChunkedAttention(nn.Module):
         return F.linear(self.mix(F.linear(h, self.inp.weight), batch, cache), self.o.weight)
 
 
+class SharedKeyValueAttention(nn.Module):
+    """Grouped-query attention over all earlier positions whose values ARE the key projections, taken before the rotation.  q | k from one
+    product without biases; rotate-half pairs over the first ``rot_dims`` channels of every q and k head; scores times ``scale``; one added
+    to the softmax denominator; output projection.
+
+    A key/value head's row is  [rotated channels as projected | the others | rotated channels, turned]  (``dim + rot_dims`` channels):
+    its first ``dim`` are the value, its last ``dim`` the key with the turned channels behind the others, and query heads have that
+    order too (scores do not depend on the order of the channels).  The projection forms the rows as they are -- the rows of W_k that
+    are rotated stand in it twice -- so one rotation in place makes them what the table keeps: a partly rotated head stores and reads
+    ``dim + rot_dims`` channels a token instead of ``2 dim``."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int, rot_dims: int, rot_base: float, scale: float):
+        super().__init__()
+        if heads % kv_heads or rot_dims % 2 or not 0 <= rot_dims <= dim:
+            raise ValueError("heads must be a multiple of kv_heads; the rotated channel count is even and within the head")
+        self.heads, self.kv_heads, self.dim, self.rot_dims, self.scale = heads, kv_heads, dim, int(rot_dims), float(scale)
+        self.head_row = dim + self.rot_dims
+        self.nq, self.nk = heads * dim, kv_heads * self.head_row
+        self.off_k = (self.nq + 7) // 8 * 8
+        self.inp = nn.Linear(width, (self.off_k + self.nk + 7) // 8 * 8, bias=False)          # q | (empty rows) | key rows
+        self.o = nn.Linear(heads * dim, width, bias=False)
+        self.register_buffer("freq", rotary_table(rot_base, rot_dims, None)[0] if rot_dims else torch.zeros(0))
+        self.register_buffer("sink", torch.zeros(heads))                                        # one added to the denominator
+        for p in self.parameters():
+            p.requires_grad_(False)
+
+    def make_cache(self, slots) -> SlotKVCache:
+        return SlotKVCache(self.nk, 0, None, 0, slots, head_row=self.head_row, key_off=self.rot_dims)
+
+    def fuse_weights(self, q, k):
+        """The input projection from the checkpoint's matrices (both [out, in])."""
+        d, r, width = self.dim, self.rot_dims, q.shape[1]
+        w = torch.zeros((self.inp.out_features, width), dtype=q.dtype, device=q.device)
+        qh, kh = q.view(self.heads, d, width), k.view(self.kv_heads, d, width)
+        w[:self.nq] = torch.cat([qh[:, r:], qh[:, :r]], dim=1).reshape(self.nq, width)
+        w[self.off_k:self.off_k + self.nk] = torch.cat([kh, kh[:, :r]], dim=1).reshape(self.nk, width)
+        return w
+
+    def forward(self, h: torch.Tensor, batch, cache: SlotKVCache) -> torch.Tensor:
+        d, r = self.dim, self.rot_dims
+        y = F.linear(h, self.inp.weight)
+        if r:
+            rotate_norm_heads_(y, batch.tok[:, 1], [HeadSegment(0, self.heads, d, d - r, r, self.freq),
+                                                    HeadSegment(self.off_k, self.kv_heads, self.head_row, d, r, self.freq)], 0.0)
+        cache.reserve(max(p + n for p, n in zip(batch.pos0, batch.n_new)), y.dtype, y.device)
+        rows = y[:, self.off_k:self.off_k + self.nk]
+        heads = rows.unflatten(1, (self.kv_heads, self.head_row))
+        ctx = sink_attend(y[:, :self.nq].unflatten(1, (self.heads, d)), heads[:, :, r:], heads[:, :, :d], cache, batch, self.scale, None, 0, self.sink)
+        cache_append(cache, rows, None, batch)
+        return F.linear(ctx, self.o.weight)
+
+
 class LatentAttention(nn.Module):
     """``rot_dim = 0``: no rotated key part (attention without positions).  ``sink`` / ``gated`` False: plain softmax / no output
-    gate.  ``own_latent`` False: the mixer has no latent projection of its own and attends over the rows of ANOTHER latent mixer of
+    gate; ``gate_channels``: the output gate is a number per channel of the concatenated heads instead of one per head.  ``q_rank``:
+    queries are products of a normed latent of their own, ``W_uq norm(W_dq h)`` (None: of h).  ``interleaved``: the rotated parts turn in
+    pairs (2i, 2i + 1) instead of (i, i + rot_dim / 2).  ``own_latent`` False: the mixer has no latent projection of its own and attends over the rows of ANOTHER latent mixer of
     the same ``kv_rank`` (and rotated part) -- the table that mixer's cache holds and the rows it formed in this step, which its
     cache hands over (``SharedLatentRows``) -- with its own queries, key and value products."""
 
     def __init__(self, width: int, heads: int, dim: int, rot_dim: int, vdim: int, kv_rank: int, rot_base: float,
-                 rot_scaling: Optional[dict], scale: float, eps: float, sink: bool = True, gated: bool = True, own_latent: bool = True):
+                 rot_scaling: Optional[dict], scale: float, eps: float, sink: bool = True, gated: bool = True, own_latent: bool = True,
+                 q_rank: Optional[int] = None, interleaved: bool = False, gate_channels: bool = False):
         super().__init__()
         if rot_dim % 2:
             raise ValueError("the rotated part has an even number of channels")
+        self.q_rank, self.interleaved, self.gate_channels = q_rank, bool(interleaved), bool(gate_channels)
         self.width, self.heads, self.dim, self.rot_dim, self.vdim, self.kv_rank = width, heads, dim, rot_dim, vdim, kv_rank
         self.scale, self.eps = float(scale), float(eps)
         self.gated, self.own_latent = bool(gated), bool(own_latent)
         self.dk = dim + rot_dim
         self.nq, self.nl = heads * self.dk, kv_rank + rot_dim
         self.n_own = self.nl if own_latent else 0
-        # q | latent, rotated key part | gate, padded with empty rows to a multiple of 8 (rows of the product start 16-byte aligned)
-        self.inp = nn.Linear(width, (self.nq + self.n_own + (heads if gated else 0) + 7) // 8 * 8, bias=False)
+        self.n_gate = (heads * vdim if self.gate_channels else heads) if gated else 0
+        # q (or its latent) | latent, rotated key part | gate; empty rows in between, so that every part starts 16-byte aligned
+        self.n_first = self.nq if q_rank is None else int(q_rank)
+        self.off_latent = (self.n_first + 7) // 8 * 8
+        self.off_gate = (self.off_latent + self.n_own + 7) // 8 * 8
+        self.inp = nn.Linear(width, (self.off_gate + self.n_gate + 7) // 8 * 8, bias=False)
+        if q_rank is not None:
+            self.uq = nn.Linear(self.n_first, self.nq, bias=False)
+            self.register_buffer("q_norm", torch.ones(self.n_first))
         # rows of every head's key product, padded with rot_dim empty rows per head (the shared rotated part is written there), then
         # the value product: one matrix product forms every head's keys and values of a whole prompt
         self.up = nn.Linear(kv_rank, heads * (self.dk + vdim), bias=False)
@@ -370,29 +445,39 @@ class LatentAttention(nn.Module):
         return SharedLatentRows(source)
 
     def fuse_weights(self, q, dkv, g, uk, uv):
-        """The module's matrices from the checkpoint's (all [out, in]); ``dkv`` / ``g`` None for a mixer without them."""
+        """The module's matrices from the checkpoint's (all [out, in]); ``q`` is W_dq of a mixer with a query latent; ``dkv`` / ``g`` None
+        for a mixer without them."""
         h, d, r, dv, rank = self.heads, self.dim, self.rot_dim, self.vdim, self.kv_rank
+        inp = torch.zeros((self.inp.out_features, q.shape[1]), dtype=q.dtype, device=q.device)
+        for off, part in ((0, q), (self.off_latent, dkv), (self.off_gate, g)):
+            if part is not None:
+                inp[off:off + part.shape[0]] = part
         uk_pad = torch.cat([uk.view(h, d, rank), torch.zeros((h, r, rank), dtype=uk.dtype, device=uk.device)], dim=1).reshape(h * (d + r), rank)
-        parts = [q] + ([dkv] if self.own_latent else []) + ([g] if self.gated else [])
-        pad = torch.zeros((self.inp.out_features - sum(p.shape[0] for p in parts), q.shape[1]), dtype=q.dtype, device=q.device)
-        return {"inp.weight": torch.cat(parts + [pad]), "up.weight": torch.cat([uk_pad, uv]),
+        return {"inp.weight": inp, "up.weight": torch.cat([uk_pad, uv]),
                 "uk_heads": uk.view(h, d, rank).contiguous(), "uv_heads_t": uv.view(h, dv, rank).transpose(1, 2).contiguous()}
 
     def forward(self, h: torch.Tensor, batch, cache) -> torch.Tensor:
         t, hd, d, r, dv, rank = h.shape[0], self.heads, self.dim, self.rot_dim, self.vdim, self.kv_rank
         y = F.linear(h, self.inp.weight)
         pos = batch.tok[:, 1]
-        segments = [HeadSegment(0, hd, self.dk, d, r, self.freq, self.rot_mult)] if r else []
+        turn = HeadSegment(0, hd, self.dk, d, r, self.freq, self.rot_mult, interleaved=self.interleaved) if r else None
+        if self.q_rank is not None:
+            segments = [HeadSegment(0, 1, self.n_first, norm=NORM_WEIGHT, weight=self.q_norm)]
+        else:
+            segments = [turn] if r else []
         if self.own_latent:
-            segments.append(HeadSegment(self.nq, 1, rank, norm=NORM_WEIGHT, weight=self.latent_norm))
+            segments.append(HeadSegment(self.off_latent, 1, rank, norm=NORM_WEIGHT, weight=self.latent_norm))
             if r:
-                segments.append(HeadSegment(self.nq + rank, 1, r, 0, r, self.freq, self.rot_mult))
+                segments.append(HeadSegment(self.off_latent + rank, 1, r, 0, r, self.freq, self.rot_mult, interleaved=self.interleaved))
         if segments:
             rotate_norm_heads_(y, pos, segments, self.eps)
-        q = y[:, :self.nq].view(t, hd, self.dk)
-        gate = y[:, self.nq + self.n_own:self.nq + self.n_own + hd] if self.gated else None
+        if self.q_rank is not None:                                                # (these queries are turned further down)
+            q = F.linear(y[:, :self.n_first], self.uq.weight).view(t, hd, self.dk)
+        else:
+            q, turn = y[:, :self.nq].view(t, hd, self.dk), None
+        gate = y[:, self.off_gate:self.off_gate + self.n_gate] if self.gated else None
         if self.own_latent:
-            latent = y[:, self.nq:self.nq + self.nl]                               # c | rotated key part: the cached row
+            latent = y[:, self.off_latent:self.off_latent + self.nl]               # c | rotated key part: the cached row
             cache.reserve(max(p + n for p, n in zip(batch.pos0, batch.n_new)), y.dtype, y.device)
             table = cache
         else:
@@ -405,12 +490,15 @@ class LatentAttention(nn.Module):
             keys = kv[:, :self.nq].view(t, hd, self.dk)
             if r:
                 keys[:, :, d:] = latent[:, None, rank:]
+            if turn is not None:
+                rotate_norm_heads_(q.flatten(1), pos, [turn], self.eps)
             ctx = sink_attend(q, keys, kv[:, self.nq:].view(t, hd, dv), None, batch, self.scale, None, 0, self.sink, gate)
         else:
-            qa = head_project(q, self.uk_heads, r)                                 # W_uk^T q | rotated part, per head
+            qa = head_project(q, self.uk_heads, r, turn, pos)                      # W_uk^T q | rotated part, per head
+            per_channel = gate if self.gate_channels else None                     # (meets the value channels, behind W_uv)
             mixed = sink_attend(qa, latent.view(t, 1, self.nl), latent[:, :rank].view(t, 1, rank), table, batch, self.scale, None, 0,
-                                self.sink, gate)
-            ctx = head_project(mixed.view(t, hd, rank), self.uv_heads_t).view(t, hd * dv)
+                                self.sink, None if self.gate_channels else gate)
+            ctx = head_project(mixed.view(t, hd, rank), self.uv_heads_t, gate=per_channel).view(t, hd * dv)
         if self.own_latent:
             cache_append(cache, latent, None, batch)
             cache.step_rows = latent                                # for mixers that attend over these rows later in the step

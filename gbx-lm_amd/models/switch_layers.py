@@ -128,35 +128,47 @@ class DenseRoutedGLU(nn.Module):
     column.  ``scoring = "sigmoid"``: scores s = sigmoid(logits); the choice runs on s + ``correction`` (a vector per
     expert that steers the choice and never the weights); with ``groups = (count, keep)`` the experts form ``count`` equal groups of
     neighbours, a group's score is the sum of its two largest choice scores and only experts of the ``keep`` best groups can be
-    chosen; weights = the chosen s, divided by their sum (+ 1e-20) if ``renormalize``, times ``route_scale``.
+    chosen; weights = the chosen s, divided by their sum (+ 1e-20) if ``renormalize``, times ``route_scale``.  ``corrected`` False: no
+    such vector (then the scores are the weights as they are: no groups, no ``renormalize``, no ``route_scale``).
     Expert e: down_e(act(gate_e h, up_e h)); ``activation = "silu"``: silu(g) u; ``"clamped_swish"``: g' = min(g, limit), u' =
     clamp(u, -limit, limit), g' sigmoid(1.702 g') (u' + 1).  ``gate_up`` stacks gate_e over up_e as [E, 2F, K], ``down`` is [E, K, F].
+    ``activation = "relu2"`` is an expert without a gate, down_e(relu(up_e h)^2): ``gate_up`` is then up_e alone, [E, F, K].
     ``forward`` returns (y [T, top, K], weights fp32 [T, top], or [T, top + 1] with ``gate_row``): the weighted sum is left to the caller, which folds it into its
-    normalisation / residual launch."""
+    normalisation / residual launch.  ``weigh_input``: an expert reads w h instead and the outputs are added as they are (``forward``
+    returns None for the weights); the weight meets the expert's first products in 32-bit, which are linear in h."""
 
     def __init__(self, input_dims: int, hidden_dims: int, num_experts: int, top: int, renormalize: bool = False, scoring: str = "softmax",
-                 groups=None, route_scale: float = 1.0, activation: str = "silu", limit: float = 0.0, gate_row: bool = False):
+                 groups=None, route_scale: float = 1.0, activation: str = "silu", limit: float = 0.0, gate_row: bool = False,
+                 weigh_input: bool = False, corrected: bool = True):
         super().__init__()
         if (gate_row or groups is not None) and scoring == "softmax" and renormalize or (gate_row and scoring != "softmax"):
             raise ValueError("softmax groups and a gate row go with probabilities as they are")
         if not 1 <= top <= num_experts:
             raise ValueError("top must lie in 1..num_experts")
-        if scoring not in ("softmax", "sigmoid") or activation not in ("silu", "clamped_swish"):
+        if scoring not in ("softmax", "sigmoid") or activation not in ("silu", "clamped_swish", "relu2"):
             raise ValueError("unknown router scoring or expert activation")
         if groups is not None and (num_experts % groups[0] or not 1 <= groups[1] <= groups[0] or top > groups[1] * (num_experts // groups[0])):
             raise ValueError("groups: equal groups, 1 <= keep <= count, and the kept groups hold at least top experts")
         self.input_dims, self.hidden_dims, self.num_experts, self.top, self.renormalize = input_dims, hidden_dims, num_experts, top, renormalize
         self.scoring, self.groups, self.route_scale = scoring, (None if groups is None else (int(groups[0]), int(groups[1]))), float(route_scale)
-        self.activation, self.limit, self.gate_row = activation, float(limit), bool(gate_row)
+        if weigh_input and gate_row:
+            raise ValueError("a gate row goes with weights on the experts' outputs")
+        self.activation, self.limit, self.gate_row, self.weigh_input = activation, float(limit), bool(gate_row), bool(weigh_input)
         self.register_buffer("router", torch.zeros((num_experts + int(self.gate_row), input_dims), dtype=torch.float32))
-        if scoring == "sigmoid":
+        self.correction = None
+        if scoring == "sigmoid" and corrected:
+            del self.correction
             self.register_buffer("correction", torch.zeros(num_experts, dtype=torch.float32))
-        self.register_buffer("gate_up", torch.zeros((num_experts, 2 * hidden_dims, input_dims)))
+        elif scoring == "sigmoid" and (groups is not None or renormalize or route_scale != 1.0):
+            raise ValueError("groups, renormalize and route_scale go with a correction")
+        self.register_buffer("gate_up", torch.zeros((num_experts, (1 if activation == "relu2" else 2) * hidden_dims, input_dims)))
         self.register_buffer("down", torch.zeros((num_experts, input_dims, hidden_dims)))
 
     def route(self, h: torch.Tensor):
         if h.is_cuda:
             from .. import mixer_ops as M
+            if self.scoring == "sigmoid" and self.correction is None:
+                return M.route_groups(h, self.router, self.num_experts, self.top, None, sigmoid=True)
             if self.scoring == "sigmoid":
                 return M.route_sigmoid_groups(h, self.router, self.correction, self.top, self.groups, self.renormalize, self.route_scale)
             if self.groups is not None or self.gate_row:
@@ -165,7 +177,7 @@ class DenseRoutedGLU(nn.Module):
         logits = F.linear(h.float(), self.router.float())
         if self.scoring == "sigmoid":
             s = torch.sigmoid(logits)
-            c = s + self.correction.float()
+            c = logits if self.correction is None else s + self.correction.float()      # (a sigmoid keeps the logits' order)
             if self.groups is not None:
                 count, keep = self.groups
                 per = c.view(c.shape[0], count, -1)
@@ -197,13 +209,18 @@ class DenseRoutedGLU(nn.Module):
 
     def forward(self, h: torch.Tensor):
         idx, w = self.route(h)
+        given = None if self.weigh_input else w
         if h.is_cuda:
             from .. import mixer_ops as M
-            return M.expert_glu(h, self.gate_up, self.down, idx, self.activation, self.limit), w
-        from .feed_forward import glu_
+            return M.expert_glu(h, self.gate_up, self.down, idx, self.activation, self.limit, w if self.weigh_input else None), given
+        from .feed_forward import activate_, glu_
         y = torch.empty((h.shape[0], self.top, self.input_dims), dtype=h.dtype, device=h.device)
         for e in range(self.num_experts):
             t, s = torch.nonzero(idx == e, as_tuple=True)
             if t.numel():
-                y[t, s] = F.linear(glu_(F.linear(h[t], self.gate_up[e]), self.activation, self.limit), self.down[e])
-        return y, w
+                z = F.linear(h[t], self.gate_up[e])
+                if self.weigh_input:
+                    z = (z.float() * w[t, s][:, None]).to(h.dtype)
+                z = activate_(z, self.activation) if self.activation == "relu2" else glu_(z, self.activation, self.limit)
+                y[t, s] = F.linear(z, self.down[e])
+        return y, given

@@ -18,12 +18,13 @@ from typing import Any, Callable, Generator, List, Optional, Tuple, Type, Union
 import torch
 from torch import nn
 
-from .models import laruzen, leripel, qdeepseek_v3, qllama, qmixtral, qphi3, qqwen2, qqwen3, qqwen3_moe, radenex, revitar, tugolix
+from .models import gibalorn, laruzen, leripel, qdeepseek_v3, qllama, qmixtral, qphi3, qqwen2, qqwen3, qqwen3_moe, radenex, revitar, tugolix
 from .models import cache as cache_mod
 from .models.quantized_linear_gba import QuantizedLinear
 from .tokenizer_utils import TokenizerWrapper, load_tokenizer
 
 MODEL_MAPPING = {
+    "gibalorn": gibalorn,     # dense checkpoint of pre-norm layers: latent, shared key/value and state space mixers, experts with weighted inputs
     "laruzen": laruzen,       # dense checkpoint in sandwich-norm form: recurrent, linear-attention and parallel mixers, named by "architecture"
     "leripel": leripel,       # dense checkpoint of parallel layers with routed experts, retention, state space and chunked attention mixers
     "llama": qllama,

@@ -82,10 +82,22 @@ int gbxm_stream_add(float* x, const void* a, const void* b, int64_t n, int32_t a
 /* The same update of rows [T][width], then h[t] = rms_norm(x[t]) * w in the activation dtype (the next layer's input). */
 int gbxm_stream_add_norm(float* x, const void* a, const void* b, const float* w, void* h, int64_t T, int32_t width, float eps, int32_t act,
                          void* stream);
-/* A matrix per head on few rows: out[t][h][j] = sum_i in[t][h][i] w[h][i][j] (j < n_out), then n_tail channels copied from
- * in[t][h][n_in ..] to out[t][h][n_out ..].  Strides in elements; w is [H][n_in][n_out]. */
-int gbxm_head_project(const void* in, int64_t in_row, int64_t in_head, const void* w, void* out, int64_t out_row, int64_t out_head, int64_t T,
-                      int32_t H, int32_t n_in, int32_t n_out, int32_t n_tail, int32_t act, void* stream);
+/* A matrix per head on few rows: out[t][h][j] = sum_i in[t][h][i] w[h][i][j] (j < n_out), times sigmoid(gate[t][h * n_out + j]) if gate is
+ * given; then n_tail channels from in[t][h][n_in ..] to out[t][h][n_out ..] -- copied, or with freq [n_tail / 2] turned by position *
+ * freq[i], cos and sin times mult (pairs i, i + n_tail / 2; or 2i, 2i+1 when interleaved).  Strides in elements; w is [H][n_in][n_out]. */
+typedef struct {
+  const void* in;   int64_t in_row, in_head;
+  const void* w;
+  void* out;        int64_t out_row, out_head;
+  const void* gate; int64_t gate_row;                 /* activation dtype, or null */
+  const int32_t* positions; int64_t pos_stride;       /* [T], with freq */
+  const float* freq;
+  int64_t T;
+  int32_t H, n_in, n_out, n_tail;
+  float mult;
+  int32_t interleaved, act;
+} gbxm_head_project_args;
+int gbxm_head_project(const gbxm_head_project_args* a, void* stream);
 /* In place on n elements, fp32 arithmetic: kind 1 = relu(z)^2, 2 = gelu in its tanh form. */
 #define GBXM_ACT_RELU2 1
 #define GBXM_ACT_GELU_TANH 2
@@ -125,7 +137,7 @@ typedef struct {
   const int32_t* tiles;         /* [n_tiles][2] (prompt kernel) */
   void* out;                    /* [T][H*dv] */
   const float* sink;            /* [H], or null: plain softmax */
-  const void* gate;  int64_t gate_row;                /* [T][H] activation dtype, or null: out *= sigmoid(gate) */
+  const void* gate;  int64_t gate_row;                /* [T][H] (or [T][H*dv]: gate_channels) activation dtype, or null: out *= sigmoid(gate) */
   int64_t T;
   int32_t B, n_tiles, q_tile;
   int32_t H, G, dk, dv;
@@ -138,6 +150,7 @@ typedef struct {
   int32_t chunk;                /* > 0: a row sees its own chunk of positions only (counted from position 0 of the sequence) */
   const float* head_scale;      /* [H], or null */
   int64_t out_row;              /* elements between output rows (0: H*dv) */
+  int32_t gate_channels;        /* the gate is a number per channel of the concatenated heads */
 } gbxm_sink_attn_args;
 int gbxm_sink_attention(const gbxm_sink_attn_args* a, void* stream);
 int gbxm_sink_attention_tiled(int32_t dk, int32_t dv, int32_t act, int32_t decode_only);
@@ -171,6 +184,23 @@ int gbxm_route_sigmoid_groups(const float* logits, const float* correction, int3
 /* gbxm_expert_glu with the expert's activation as a parameter (GBXM_GLU_*, alpha = 1.702 for kind 2). */
 int gbxm_expert_glu_act(const void* h, const void* gate_up, const void* down, const int32_t* idx, void* y, int64_t T, int32_t K, int32_t F,
                         int32_t E, int32_t top, int32_t act, int32_t kind, float limit, void* ws, size_t ws_bytes, void* stream);
+
+/* The same with every parameter named.  kind GBXM_EXPERT_RELU2: experts without a gate, y = down[e] relu(up[e] h)^2, `first` [E][F][K].
+ * scale (or null) [T][top]: an expert reads scale * h -- the factor meets the sums of its first products, in fp32. */
+#define GBXM_EXPERT_RELU2 16
+typedef struct {
+  const void* h;
+  const void* first;            /* [E][2F][K] gate over up, or [E][F][K] */
+  const void* down;             /* [E][K][F] */
+  const int32_t* idx;           /* [T][top] */
+  const float* scale;
+  void* y;                      /* [T][top][K] */
+  int64_t T;
+  int32_t K, F, E, top, act, kind;
+  float limit;
+  void* ws; size_t ws_bytes;    /* gbxm_expert_glu_workspace */
+} gbxm_expert_args;
+int gbxm_expert_ff(const gbxm_expert_args* a, void* stream);
 
 /* ---- recurrent mixers: a decayed matrix state per head (gbx-lm_amd/models/recurrent_mixers.py) ---- */
 
@@ -302,8 +332,8 @@ int gbxm_gate_group_norm(const float* o, const void* z, int64_t z_stride, const 
 /* ---- parallel layers with routed experts (gbx-lm_amd/models/residual.py:layer_update_, models/switch_layers.py) ---- */
 
 /* v = (replace ? 0 : x[t]) + branch[t] + sum_{k < top} mix[t * mix_row + k] cand[t][k] + extra[t];  x[t] <- v;  image[t] = v in the activation
- * dtype (row stride image_row);  h[t] = rms_norm(v) * norm_w in the activation dtype.  cand / extra / image / norm_w may be null;
- * top <= 64. */
+ * dtype (row stride image_row);  h[t] = rms_norm(v) * norm_w in the activation dtype.  image / norm_w may be null, and of branch / cand /
+ * extra all but one; mix null: weights of 1; top <= 64. */
 typedef struct {
   float* x;
   const void* branch; int64_t branch_row;
@@ -321,11 +351,11 @@ typedef struct {
 int gbxm_layer_update(const gbxm_layer_update_args* a, void* stream);
 /* logits[t][e] = sum_k h[t][k] router[e][k] in fp32, for few rows. */
 int gbxm_router_rows(const void* h, const float* router, float* logits, int64_t T, int32_t K, int32_t E, int32_t act, void* stream);
-/* Router decisions from fp32 logit rows (stride `row`): s = softmax over E; with n_groups > 0 only experts of the keep_groups groups (equal
+/* Router decisions from fp32 logit rows (stride `row`): s = softmax over E -- or, with `sigmoid` (no groups, no gate), the sigmoid of each; with n_groups > 0 only experts of the keep_groups groups (equal
  * groups of neighbours) with the largest s in them; the `top` largest s (ties: lower index), weights = s as they are.  gate: logit E of a
  * row is a gate's, weight[top] = its sigmoid. */
 int gbxm_route_groups(const float* logits, int64_t row, int32_t* idx, float* weight, int64_t weight_row, int64_t T, int32_t E, int32_t top,
-                      int32_t n_groups, int32_t keep_groups, int32_t gate, void* stream);
+                      int32_t n_groups, int32_t keep_groups, int32_t gate, int32_t sigmoid, void* stream);
 
 #ifdef __cplusplus
 }
