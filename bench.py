@@ -776,6 +776,41 @@ def laruzen_bench(args):
     print(json.dumps({"metric": "laruzen_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "sizes": out}))
 
 
+def ragged_legs(model, vocab, tag, res, name=None):
+    """Prefill (one scheduler step of a whole prompt) and decode (scheduler steps, HIP-graph replay from the third on) throughput of a
+    ragged-step model into ``res`` under ``tag``."""
+    from gbx_lm_amd.batching import BatchScheduler
+
+    def clock(fn, reps, untimed=2):                  # (the second call of a shape still pays one-time allocations)
+        for _ in range(untimed):
+            fn()
+        torch.cuda.synchronize()
+        e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+        e0.record()
+        for _ in range(reps):
+            fn()
+        e1.record()
+        torch.cuda.synchronize()
+        return e0.elapsed_time(e1) / reps
+
+    toks = lambda n, o=0: [(o + i * 7919) % vocab for i in range(n)]
+    for T in (512, 4096):
+        def prefill():
+            eng = BatchScheduler(model)
+            eng.step([("p", toks(T))])
+        res[f"{tag}prefill_T{T}_tok_s"] = round(T / clock(prefill, 3) * 1e3)
+    for B, ctx in ((1, 2048), (32, 256)):
+        eng = BatchScheduler(model)
+        eng.step([(i, toks(ctx, i)) for i in range(B)])
+        state = {"t": 0}
+        def decode():
+            state["t"] += 1
+            eng.step([(i, [(state["t"] * 31 + i) % vocab]) for i in range(B)])
+        res[f"{tag}decode_B{B}_ctx{ctx}_tok_s"] = round(B / clock(decode, 64, 6) * 1e3)         # (the third step captures the graph)
+        del eng
+    print(tag or name, res, file=sys.stderr, flush=True)
+
+
 LERIPEL_SIZES = {
     # name: Leripel geometry (r retention, m state space mixer, a chunked attention; routed experts with a gated shared one in every layer)
     # and, from it, the Laruzen (the closest existing model: dense bf16 decoder over ragged steps with linear-attention states, attention
@@ -798,39 +833,8 @@ def leripel_bench(args):
     Laruzen of equal width, layer runs, routed experts and state geometry.  One JSON line; the default workload of
     this file is untouched."""
     from gbx_lm_amd import synthetic as S
-    from gbx_lm_amd.batching import BatchScheduler
     dev = torch.device("cuda", 0)
     torch.cuda.set_device(dev)
-
-    def clock(fn, reps, untimed=2):                  # (the second call of a shape still pays one-time allocations)
-        for _ in range(untimed):
-            fn()
-        torch.cuda.synchronize()
-        e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
-        e0.record()
-        for _ in range(reps):
-            fn()
-        e1.record()
-        torch.cuda.synchronize()
-        return e0.elapsed_time(e1) / reps
-
-    def legs(model, vocab, tag, res):
-        toks = lambda n, o=0: [(o + i * 7919) % vocab for i in range(n)]
-        for T in (512, 4096):
-            def prefill():
-                eng = BatchScheduler(model)
-                eng.step([("p", toks(T))])
-            res[f"{tag}prefill_T{T}_tok_s"] = round(T / clock(prefill, 3) * 1e3)
-        for B, ctx in ((1, 2048), (32, 256)):
-            eng = BatchScheduler(model)
-            eng.step([(i, toks(ctx, i)) for i in range(B)])
-            state = {"t": 0}
-            def decode():
-                state["t"] += 1
-                eng.step([(i, [(state["t"] * 31 + i) % vocab]) for i in range(B)])
-            res[f"{tag}decode_B{B}_ctx{ctx}_tok_s"] = round(B / clock(decode, 64, 6) * 1e3)         # (the third step captures the graph)
-            del eng
-        print(tag or "leripel", res, file=sys.stderr, flush=True)
 
     out = {}
     for name in args.sizes.split(","):
@@ -838,7 +842,7 @@ def leripel_bench(args):
         res = {"geometry": g}
         cfg = S.leripel_config(**g)
         model = S.build_leripel(cfg, device=dev, seed=0)
-        legs(model, cfg["vocab"], "", res)
+        ragged_legs(model, cfg["vocab"], "", res, "leripel")
         runs = [cfg["layers"][i]["type"] for i in model.layer_runs]
         del model
         torch.cuda.empty_cache()
@@ -849,19 +853,64 @@ def leripel_bench(args):
                                               moe=dict(experts=e["experts"], top=e["top"], ff=e["ff"], shared=e["shared"]),
                                               pattern="".join({"retention": "l", "mamba2": "g", "attention": "p"}[k] for k in runs), vocab=cfg["vocab"]),
                              device=dev, seed=0)
-        legs(lm, cfg["vocab"], "laruzen_", res)
+        ragged_legs(lm, cfg["vocab"], "laruzen_", res)
         del lm
         torch.cuda.empty_cache()
         out[name] = res
     print(json.dumps({"metric": "leripel_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "sizes": out}))
 
 
+GIBALORN_SIZES = {
+    # name: Gibalorn geometry (m state space mixer, l latent attention, a attention whose values are its keys; routed experts without a gate
+    # in every layer) and, from it, the Leripel (the closest existing model: dense bf16 decoder over ragged steps with state space mixers,
+    # grouped-query attention and routed experts) of equal width, layer runs and experts: the same state space mixer for m, attention over
+    # the whole context with the attention's / the latent mixer's heads for a and l
+    "small": dict(width=1024, latent=dict(heads=8, dim=64, rot_dim=32, vdim=64, kv_rank=256, q_rank=384),
+                  mamba2=dict(heads=32, vdim=64, state=128, groups=1, conv=4, norm_groups=1), attention=dict(heads=16, kv_heads=4, dim=64, rot_dims=32),
+                  moe=dict(experts=32, top=4, ff=512), pattern="mlal"),
+    "a3b-like": dict(width=2048, latent=dict(heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=1024),
+                     mamba2=dict(heads=64, vdim=64, state=128, groups=8, conv=4, norm_groups=8), attention=dict(heads=16, kv_heads=4, dim=128, rot_dims=64),
+                     moe=dict(experts=128, top=8, ff=768), pattern="mlal"),
+    "looped": dict(width=2048, latent=dict(heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=768),
+                   mamba2=dict(heads=64, vdim=64, state=128, groups=1, conv=4, norm_groups=1), attention=dict(heads=16, kv_heads=2, dim=128, rot_dims=128),
+                   moe=dict(experts=64, top=2, ff=2048), pattern="mla", loop=(0, 2, 2)),
+}
+
+
+def gibalorn_bench(args):
+    """``--design gibalorn``: prefill and decode throughput of Gibalorn at layer sizes of real models (random weights, bf16), beside
+    Leripel of equal width, layer runs, routed experts and mixer geometry.  One JSON line; the default workload of
+    this file is untouched."""
+    from gbx_lm_amd import synthetic as S
+    dev = torch.device("cuda", 0)
+    torch.cuda.set_device(dev)
+    out = {}
+    for name in args.sizes.split(","):
+        g = GIBALORN_SIZES[name]
+        res = {"geometry": g}
+        cfg = S.gibalorn_config(**g)
+        model = S.build_gibalorn(cfg, device=dev, seed=0)
+        ragged_legs(model, cfg["vocab"], "", res, "gibalorn")
+        runs = "".join({"mamba2": "m", "latent_attention": "a", "attention": "a"}[cfg["layers"][i]["type"]] for i in model.layer_runs)
+        del model
+        torch.cuda.empty_cache()
+        a, e = g["attention"], g["moe"]
+        lm = S.build_leripel(S.leripel_config(width=g["width"], retention=dict(heads=1, dim=8, vdim=8), mamba2=g["mamba2"],
+                                              attention=dict(heads=a["heads"], kv_heads=a["kv_heads"], dim=a["dim"], vdim=a["dim"], chunk=8192, rot_dims=a["rot_dims"]),
+                                              moe=dict(experts=e["experts"], top=e["top"], ff=e["ff"]), pattern=runs, vocab=cfg["vocab"]), device=dev, seed=0)
+        ragged_legs(lm, cfg["vocab"], "leripel_", res)
+        del lm
+        torch.cuda.empty_cache()
+        out[name] = res
+    print(json.dumps({"metric": "gibalorn_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "sizes": out}))
+
+
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", default=None, choices=["revitar", "radenex", "tugolix", "laruzen", "leripel"], help="side benchmark of one model design beside the closest existing "
+    ap.add_argument("--design", default=None, choices=["revitar", "radenex", "tugolix", "laruzen", "leripel", "gibalorn"], help="side benchmark of one model design beside the closest existing "
                     "family at equal size (own JSON line; the default workload and its output are unchanged)")
     ap.add_argument("--sizes", default=None, help="--design: comma-separated names of REVITAR_SIZES (default small,a3b-like) / RADENEX_SIZES "
-                    "(default small,lite-like) / TUGOLIX_SIZES / LARUZEN_SIZES / LERIPEL_SIZES (default small,a3b-like)")
+                    "(default small,lite-like) / TUGOLIX_SIZES / LARUZEN_SIZES / LERIPEL_SIZES / GIBALORN_SIZES (default small,a3b-like)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=512, help="timed decode steps (default: > 0.5 s of GPU time, so that a coarse GPU-busy sampler sees the run)")
     ap.add_argument("--warmup", type=int, default=8)
@@ -880,9 +929,10 @@ def main():
     if args.design is not None:
         if not torch.cuda.is_available():
             raise SystemExit("bench.py needs an MI355X")
-        args.sizes = args.sizes or {"revitar": "small,a3b-like", "radenex": "small,lite-like", "tugolix": "small,a3b-like", "laruzen": "small,a3b-like", "leripel": "small,a3b-like"}[args.design]
+        args.sizes = args.sizes or {"revitar": "small,a3b-like", "radenex": "small,lite-like", "tugolix": "small,a3b-like", "laruzen": "small,a3b-like", "leripel": "small,a3b-like",
+                                   "gibalorn": "small,a3b-like"}[args.design]
         return {"revitar": revitar_bench, "radenex": radenex_bench, "tugolix": tugolix_bench, "laruzen": laruzen_bench,
-                "leripel": leripel_bench}[args.design](args)
+                "leripel": leripel_bench, "gibalorn": gibalorn_bench}[args.design](args)
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:
         spawn_ranks(args.gpus)                                     # never returns; nothing has touched the GPU yet
     world = int(os.environ.get("WORLD_SIZE", "1"))

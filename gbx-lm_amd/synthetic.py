@@ -669,3 +669,87 @@ def build_leripel(config: Dict, device="cpu", seed: int = 0, act_dtype=torch.bfl
         raise ValueError(f"tensors without a place in the model: {skipped[:3]}")
     model.eval()
     return model
+
+
+# ------------------------------------------------------------------------------------------------ Gibalorn (latent, shared key/value and state space mixers; weighted expert inputs)
+def gibalorn_config(width: int, latent: Dict, mamba2: Dict, attention: Dict, moe: Dict, pattern: str = "mlal", loop=None, vocab: int = 32000) -> Dict:
+    """config.json of a Gibalorn model: ``pattern`` names the layers in order ('l' latent attention, 'm' state space, 'a' attention whose
+    values are its keys).  ``latent``: heads, dim, rot_dim, vdim, kv_rank, q_rank; ``mamba2``: heads, vdim, state, groups, conv,
+    norm_groups; ``attention``: heads, kv_heads, dim, rot_dims; ``moe``: experts, top, ff; ``loop``: (start, stop, times) or None."""
+    routed = {"kind": "moe", "expert": {"ff": moe["ff"]}, "router": {"experts": moe["experts"], "top": moe["top"]}}
+    layers = []
+    for c in pattern:
+        if c == "l":
+            layer = {"type": "latent_attention", "mixer": dict({k: latent[k] for k in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank")},
+                                                               scale=(latent["dim"] + latent["rot_dim"]) ** -0.5, rot={"base": 1e6, "dims": latent["rot_dim"]})}
+        elif c == "m":
+            layer = {"type": "mamba2", "mixer": {k: mamba2[k] for k in ("heads", "vdim", "state", "groups", "conv", "norm_groups")}}
+        elif c == "a":
+            d = attention["dim"]
+            layer = {"type": "attention", "mixer": {"heads": attention["heads"], "kv_heads": attention["kv_heads"], "dim": d, "vdim": d, "scale": d ** -0.5,
+                                                    "rot": {"base": 1e6, "dims": attention["rot_dims"]}}}
+        else:
+            raise ValueError(f"gibalorn_config: unknown layer letter {c!r}")
+        layers.append(dict(layer, mlp=json.loads(json.dumps(routed))))
+    return {"architecture": "Gibalorn", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": layers,
+            "loop": None if loop is None else {"start": loop[0], "stop": loop[1], "times": loop[2]}}
+
+
+def gibalorn_checkpoint(config: Dict, device="cpu", seed: int = 0, dtype=torch.bfloat16) -> Dict[str, torch.Tensor]:
+    """Random tensors in the design's checkpoint names with real shapes, generated directly on ``device``."""
+    device = torch.device(device)
+    gen = torch.Generator(device=device)
+    gen.manual_seed(seed)
+    W = config["width"]
+
+    def mat(o, i, mult=1.0):
+        return (torch.randn((o, i), device=device, generator=gen) * (mult * i ** -0.5)).to(dtype)
+
+    def vec(n, lo, hi):
+        return (torch.rand((n,), device=device, generator=gen) * (hi - lo) + lo).to(dtype)
+
+    w = {"embed": torch.randn((config["vocab"], W), device=device, generator=gen).to(dtype), "final.norm": vec(W, 0.9, 1.1), "head": mat(config["vocab"], W)}
+    for i, layer in enumerate(config["layers"]):
+        p, m, kind = f"l{i}.", layer["mixer"], layer["type"]
+        w[p + "norm1"] = vec(W, 0.9, 1.1)
+        x, H, dv = p + "mix.", m["heads"], m["vdim"]
+        w[x + "o"] = mat(W, H * dv)
+        if kind == "mamba2":
+            inner, gn = H * dv, m["groups"] * m["state"]
+            w[x + "in"] = mat(2 * inner + 2 * gn + H, W)
+            w[x + "conv"], w[x + "conv.b"] = (torch.randn((inner + 2 * gn, m["conv"]), device=device, generator=gen) * 0.5 + 0.25).to(dtype), vec(inner + 2 * gn, -0.1, 0.1)
+            w[x + "dt_bias"], w[x + "A_log"], w[x + "D"], w[x + "norm"] = vec(H, -4.0, -1.0), vec(H, 0.0, 2.0), vec(H, 0.5, 1.0), vec(inner, 0.9, 1.1)
+        elif kind == "latent_attention":
+            d, r, rank, qr = m["dim"], m["rot_dim"], m["kv_rank"], m["q_rank"]
+            w[x + "dq"], w[x + "dq.norm"], w[x + "uq"] = mat(qr, W), vec(qr, 0.9, 1.1), mat(H * (d + r), qr)
+            w[x + "dkv"], w[x + "dkv.norm"] = mat(rank + r, W), vec(rank, 0.9, 1.1)
+            w[x + "uk"], w[x + "uv"], w[x + "g"] = mat(H * d, rank), mat(H * dv, rank), mat(H * dv, W)
+        else:
+            w[x + "q"], w[x + "k"] = mat(H * m["dim"], W), mat(m["kv_heads"] * m["dim"], W)
+        ff = layer.get("mlp")
+        if ff is not None:
+            f, n, E = p + "mlp.", ff["expert"]["ff"], ff["router"]["experts"]
+            w[p + "norm2"], w[f + "router"] = vec(W, 0.9, 1.1), mat(E, W, 2.0)
+            for e in range(E):
+                w[f + f"e{e}.up"], w[f + f"e{e}.down"] = mat(n, W), mat(W, n)
+    return w
+
+
+def build_gibalorn(config: Dict, device="cpu", seed: int = 0, act_dtype=torch.bfloat16):
+    """Random-init Gibalorn with real shapes: a random checkpoint generated on ``device`` goes through the model's own ``sanitize``."""
+    from .models import gibalorn
+    from .utils import load_weights
+    device = torch.device(device)
+    weights = gibalorn_checkpoint(config, device, seed)
+    args = gibalorn.ModelArgs.from_dict(config)
+    model = gibalorn.Model(args)                  # (the buffers the constructors compute -- frequency tables, sinks -- are tiny)
+    weights = model.sanitize(weights)
+    weights = {k: (v.to(act_dtype) if v.is_floating_point() and v.dtype != torch.float32 else v) for k, v in weights.items()}
+    with torch.device("meta"):
+        model = gibalorn.Model(args)
+    model = model.to_empty(device=device)
+    skipped = load_weights(model, weights, device=device)
+    if skipped:
+        raise ValueError(f"tensors without a place in the model: {skipped[:3]}")
+    model.eval()
+    return model
