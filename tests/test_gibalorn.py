@@ -447,9 +447,9 @@ def test_attention_gates_per_channel(device, dtype):
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("rows,experts,top,ff,width", [(5, 6, 1, 24, 64), (70, 8, 3, 40, 48), (300, 5, 2, 96, 64), (300, 3, 3, 32, 160), (90, 130, 4, 64, 32), (3, 4, 2, 7, 37),
-                                                       (130, 4, 2, 7, 37), (512, 9, 1, 288, 96)])
+                                                       (130, 4, 2, 7, 37), (512, 9, 1, 288, 96), (64, 6, 2, 96, 160), (40, 3, 2, 32, 32)])
 def test_experts_that_read_weighted_inputs(device, dtype, rows, experts, top, ff, width):
-    """Row kernels and grouped matrix-core products (256 pairs and more on the 32-grid); the weight inside the square of relu, not on the
+    """Row kernels and both forms of grouped matrix-core products (64 pairs and more on the 32-grid, few or many per expert); the weight inside the square of relu, not on the
     output; the choice of every row against the oracle's where no close call decides it."""
     g = torch.Generator().manual_seed(6)
     m = DenseRoutedGLU(width, ff, experts, top, scoring="sigmoid", activation="relu2", weigh_input=True, corrected=False)
@@ -476,7 +476,7 @@ def test_gated_experts_read_weighted_inputs_too(device):
     """The input's weight is a parameter of the routed experts: silu experts behind the same router, few rows and many, fp32 and bf16."""
     g = torch.Generator().manual_seed(7)
     for dtype in DTYPES:
-        for rows in (4, 200):
+        for rows in (4, 60, 200):
             m = DenseRoutedGLU(64, 32, 4, 2, scoring="sigmoid", weigh_input=True, corrected=False)
             m.router = torch.randn(m.router.shape, generator=g) * 0.125
             m.gate_up, m.down = (torch.randn(m.gate_up.shape, generator=g) * 0.125).to(dtype), (torch.randn(m.down.shape, generator=g) * 0.2).to(dtype)
