@@ -24,7 +24,7 @@ constexpr int NT = 256, NW = NT / 64;
 constexpr int KT = 64;            // keys per tile
 constexpr int RC = 8;             // query heads a workgroup takes at most
 constexpr int DCH = 128;          // value channels per lane pass (two per lane)
-constexpr int NCH = 4;            // lane passes: value sizes up to NCH * DCH
+constexpr int NCH_MAX = 8;        // lane passes: value sizes up to NCH_MAX * DCH (a kernel is compiled for 4 and for 8)
 
 struct SinkGeo {
   int H, G, dk, dv, window, keep, ring, chunk, gate_channels;
@@ -58,7 +58,7 @@ __device__ __forceinline__ float dot_row(const float* __restrict__ q, const T* _
   return dot;
 }
 
-template <typename T, bool FAST, bool VEC>
+template <typename T, bool FAST, bool VEC, int NCH>
 __global__ __launch_bounds__(NT) void sink_rows_kernel(const T* __restrict__ q, const T* __restrict__ kn, const T* __restrict__ vn,
                                                       const T* __restrict__ kc, const T* __restrict__ vc, const int* __restrict__ seq,
                                                       const int* __restrict__ tok, T* __restrict__ out, const float* __restrict__ sink,
@@ -289,10 +289,14 @@ int launch_rows(const gbxm_sink_attn_args& a, const SinkGeo& g, int rc, int chun
   const T* gate = static_cast<const T*>(a.gate);
   T* out = static_cast<T*>(a.out);
   float* part = static_cast<float*>(a.partial);
-  if (vec)
-    sink_rows_kernel<T, FAST, true><<<grid, NT, lds, s>>>(q, kn, vn, kc, vc, a.seq, a.tok, out, a.sink, gate, g, rc, splits, part);
-  else
-    sink_rows_kernel<T, FAST, false><<<grid, NT, lds, s>>>(q, kn, vn, kc, vc, a.seq, a.tok, out, a.sink, gate, g, rc, splits, part);
+  auto go = [&](auto kernel) { kernel<<<grid, NT, lds, s>>>(q, kn, vn, kc, vc, a.seq, a.tok, out, a.sink, gate, g, rc, splits, part); };
+  if (a.dv <= 4 * DCH) {
+    if (vec) go(sink_rows_kernel<T, FAST, true, 4>);
+    else go(sink_rows_kernel<T, FAST, false, 4>);
+  } else {
+    if (vec) go(sink_rows_kernel<T, FAST, true, NCH_MAX>);
+    else go(sink_rows_kernel<T, FAST, false, NCH_MAX>);
+  }
   if (splits > 1) sink_reduce_kernel<T, FAST><<<dim3(a.T, a.H), 256, 0, s>>>(part, out, a.sink, gate, a.gate_row, a.gate_channels, a.T, a.H, a.dv, splits,
                                                                                        g.out_row);
   return after_launch("sink_attention (rows)");
@@ -821,7 +825,7 @@ int gbxm_sink_attention(const gbxm_sink_attn_args* a, void* stream) {
             a->out_row > 0 ? a->out_row : static_cast<int64_t>(a->H) * a->dv, a->q_row, a->q_head, a->k_row, a->k_head, a->v_row, a->v_head,
             a->kc_slot, a->kc_row, a->kc_head, a->vc_slot, a->vc_row, a->vc_head, a->gate_row};
   const int R = a->H / a->G;
-  if (a->dv > NCH * DCH) return fail(GBXM_ERR_UNSUPPORTED, "sink_attention: value size %d beyond the row kernel (%d)", a->dv, NCH * DCH);
+  if (a->dv > NCH_MAX * DCH) return fail(GBXM_ERR_UNSUPPORTED, "sink_attention: value size %d beyond the row kernel (%d)", a->dv, NCH_MAX * DCH);
   auto lds_of = [&](int rc_) {
     return static_cast<size_t>(2 * KT) * sizeof(void*) + static_cast<size_t>(rc_) * (a->dk + KT + 3 + NW * a->dv) * sizeof(float);
   };

@@ -171,6 +171,7 @@ def dirty(cache, dtype, device):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("layer", [O.latent_layer(3, 20, 12, 24, 40, 28, 300.0, 0.2), O.latent_layer(16, 32, 16, 16, 64, 48), O.latent_layer(1, 7, 2, 5, 9, 3),
                                    O.latent_layer(2, 96, 32, 64, 272, 136), O.latent_layer(40, 8, 8, 8, 32, 2000),
+                                   O.latent_layer(2, 16, 8, 16, 600, 24),
                                    O.attention_layer(4, 2, 24, 16, 500.0, 0.3), O.attention_layer(3, 3, 10, 6), O.attention_layer(2, 1, 16, 16),
                                    O.attention_layer(4, 1, 64, 0), O.attention_layer(6, 3, 64, 32, 1e6), O.attention_layer(8, 2, 128, 64), O.attention_layer(40, 1, 32, 8),
                                    O.mamba2_layer(4, 8, 24, 2, 3, 4), O.mamba2_layer(3, 20, 10, 1, 1, 1), O.mamba2_layer(2, 72, 136, 2, 5, 3)],
